@@ -221,10 +221,11 @@ class CacheManager:
         g, i = self._group_of_entry[entry]
         return {name: pool[i] for name, pool in self.groups[g].pools.items()}
 
-    def state_of(self, entry: int):
+    def state_of(self, entry: int, name: Optional[str] = None):
         """What stop `entry` keeps per request, [slot][*shape]: the tensor of a stop that declared one
-        `StateSpec`, a dict by name of a stop that declared several."""
-        return self.state_tensors[entry]
+        `StateSpec`, a dict by name of a stop that declared several; with `name`, the tensor of that name."""
+        held = self.state_tensors[entry]
+        return held[name] if name is not None and isinstance(held, dict) else held
 
     def _state_tensors(self):
         for held in self.state_tensors.values():

@@ -35,6 +35,7 @@ class NormSpec(PartSpec):
     kind: str = "rmsnorm"
     weight_name: str = "weight"  # the tensor's name below the norm's prefix
     weight_offset: float = 0.0   # the stored tensor plus this is the weight (1: a weight stored around zero)
+    one_weight: bool = False     # the tensor is a single number (shape []), the weight of every feature
 
 
 @dataclass(frozen=True)
@@ -67,8 +68,8 @@ class WavelengthRamp:
 class PositionSpec(PartSpec):
     """Rotation of query and key by absolute position; `rotary_dim` leading
     features of each head are rotated in pairs: (i, i + rotary_dim/2) for kind
-    "neox_rope", (2i, 2i + 1) for kind "interleaved_rope" (which also takes a `ramp`:
-    a `FrequencyRamp` or a `WavelengthRamp`)."""
+    "neox_rope", (2i, 2i + 1) for kind "interleaved_rope".  `ramp`: frequencies stretched
+    by a `FrequencyRamp` or a `WavelengthRamp`."""
 
     rotary_dim: int = 0
     theta: float = 10000.0
@@ -171,6 +172,7 @@ class LatentMixerSpec(PartSpec):
     sinks: bool = False        # one learned number per head joins the softmax's denominator as exp(sink), unscaled
     sink_name: str = "sink"
     own_kv: bool = True        # False: no down projection and no norm of its own; the layer reads another stop's rows
+    gate_name: Optional[str] = None  # a projection W_g [heads, hidden] of the mixer's input: head j *= sigmoid(W_g x)_j before W_o
 
 
 @dataclass(frozen=True)
@@ -261,6 +263,40 @@ class LinearAttentionSpec(PartSpec):
     norm_name: str = "norm"
     bias_suffix: str = ".b"
     weight_suffix: str = ""
+
+
+@dataclass(frozen=True)
+class FixedDecaySpec(PartSpec):
+    """Linear attention with a fixed decay per head (lightning attention): S <- decays[h] S + k_t v_t^T, o_t = S^T q_t
+    with q = act(W_q h), k = act(W_k h), v = act(W_v h), act = `activation`; all heads' read-outs are RMS-normed
+    together with a weight [num_heads * value_dim], gated by `gate_activation`(W_g h) and projected out."""
+
+    hidden_size: int = 0
+    num_heads: int = 0
+    key_dim: int = 0
+    value_dim: int = 0
+    decays: Tuple[float, ...] = ()
+    norm_eps: float = 1e-6
+    activation: str = "silu"
+    gate_activation: str = "sigmoid"   # or "silu"
+    kind: str = "fixed_decay_linear_attention"
+    q_name: str = "q"
+    k_name: str = "k"
+    v_name: str = "v"
+    gate_name: str = "g"
+    o_name: str = "o"
+    norm_name: str = "norm"
+    weight_suffix: str = ""
+
+
+@dataclass(frozen=True)
+class InputConvSpec:
+    """What a sublayer reads is the stream plus a causal convolution of it over time, per channel:
+    h_t + sum_j w[:, j] h_(t - taps + 1 + j), zeros before the sequence's first token.  The tensors `names`
+    (mixer's, feed-forward's) are [hidden, taps]."""
+
+    taps: int
+    names: Tuple[str, str]
 
 
 @dataclass(frozen=True)
@@ -363,6 +399,7 @@ class LayerSpec:
     feed_forward_norm_prefix: str = "post_attention_layernorm."
     arrangement: str = "prenorm"
     residual_scale: float = 1.0  # what a branch is multiplied by before it joins the stream ("branchnorm")
+    input_conv: Optional[InputConvSpec] = None  # the sublayers read the stream through a convolution ("branchnorm")
     # arrangement "hyper": the stream is `streams` copies joined by hyper-connections whose tensors
     # (in [S], out [S], mix [S, S] indexed [from, to]) lie under `connection_prefixes` (mixer, feed-forward;
     # None: the plain sum x <- x + y), and a branch's output is first multiplied, feature by feature, by
@@ -429,6 +466,8 @@ class ModelPlan:
                     f"schedule entry {i} reads the cache of entry {entry.cache_from}, "
                     "which is not an earlier entry")
         for i, layer in enumerate(self.layers):
+            if layer.input_conv is not None and layer.arrangement != "branchnorm":
+                raise ConfigError(f"layer {i}: only the arrangement 'branchnorm' reads its input through a convolution")
             if layer.streams != self.streams:
                 raise ConfigError(f"layer {i} keeps {layer.streams} copies of the stream, the model {self.streams}")
             if layer.streams != 1 and layer.arrangement != "hyper":

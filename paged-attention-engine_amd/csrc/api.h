@@ -68,8 +68,8 @@ int pae_paged_attention_masked(int dtype, void* out, int64_t out_stride, const v
                                const void* k_cache, const void* v_cache, const int* positions, const int* tok_seq,
                                const int* block_tables, int max_blocks, int bs, int num_tokens, int nh, int nkv, int hd,
                                int vd, float scale, int window, float cap, const float* sinks, int chunked,
-                               const float* slopes, const void* gate, int64_t gate_stride, int shared_kv,
-                               hipStream_t stream);
+                               const float* slopes, const void* gate, int64_t gate_stride, int gate_per_head,
+                               int shared_kv, hipStream_t stream);
 // a stream kept as several copies joined by hyper-connections: see hyper.hip
 int pae_hyper_norm(int dtype, float* streams, int num_streams, const void* y, int parts, int64_t part_stride,
                    const void* ls, int ls_is_f32, const float* mix, const float* outw, const float* inw,
@@ -86,8 +86,8 @@ int pae_conv_norm_store(int dtype, const void* proj, int64_t row_stride, void* q
 // rows [q heads of (nope + rd) | latent + rd]: latent norm, rotation, write of the latent pages: see latent.hip
 int pae_latent_prepare(int dtype, const void* proj, int64_t row_stride, void* q_full, int64_t qf_stride, int num_tokens,
                        int nh, int nope, int rd, int rot, int interleaved, int rank, const void* norm_w, int w_is_f32,
-                       float eps, const float* cos_sin, const int* positions, const int* tok_seq, const int* block_tables,
-                       int max_blocks, int bs, void* latent, void* latent_t, hipStream_t stream);
+                       float eps, const float* cos_sin, float magnitude, const int* positions, const int* tok_seq,
+                       const int* block_tables, int max_blocks, int bs, void* latent, void* latent_t, hipStream_t stream);
 int pae_heads_product_few(void* out, int64_t ldc, int64_t head_c, const void* a, int64_t lda, int64_t head_a, const void* w,
                           int M, int N, int K, int heads, hipStream_t stream);  // bfloat16, a few rows, one product per head
 // latent attention on the matrix cores: see attention_latent.hip
@@ -96,7 +96,8 @@ int pae_latent_attn_columns(int H, int ct);
 int pae_latent_attn_bf16(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* latent,
                          const void* latent_t, const int* tiles, int num_tiles, int ct, const int* positions,
                          const int* block_tables, int max_blocks, int bs, int H, int kd, int C, float scale, int window,
-                         int chunked, float* part_acc, float* part_ml, const float* sinks, hipStream_t stream);
+                         int chunked, float* part_acc, float* part_ml, const float* sinks, const void* head_gate,
+                         int64_t gate_stride, hipStream_t stream);
 int pae_latent_attn_split();
 // rows [q | k | v]: RMS norm of q and of k over the whole projection, or head by head with one weight that the
 // heads share (`per_head`; weights null: none), rotation, cache write
@@ -147,6 +148,24 @@ int pae_linear_attention_step(int dtype, const void* proj, int64_t row_stride, c
                               int D, int V, float* state, int64_t state_slot_stride, const void* norm_w, int w_is_f32,
                               float norm_eps, float* work, void* out, hipStream_t stream);
 int64_t pae_linear_attention_work_floats(int num_tokens, int H, int D, int V);
+// linear attention with a fixed decay per head over a step's projected rows: see fixed_decay.hip
+int pae_fixed_decay_chunk(int D);
+int pae_fixed_decay_step(int dtype, const void* proj, int64_t row_stride, const void* gate_in, int64_t gate_stride,
+                         int gate_sigmoid, int silu, int num_tokens, const int* serial, int num_serial, const int* chunks,
+                         int num_chunks, const int* scans, int num_scans, const int* slots, const float* powers, int H,
+                         int D, int V, float* state, int64_t slot_stride, const void* norm_w, int w_is_f32, float norm_eps,
+                         float* work, void* out, hipStream_t stream);
+int64_t pae_fixed_decay_work_floats(int num_tokens, int num_chunks, int H, int D, int V);
+// the stream through a short convolution over time, as a sublayer's input: see input_conv.hip
+int pae_input_conv_tile_rows(int taps);
+int pae_input_conv(int dtype, void* rows, const float* x, const float* filters, float* ring, int64_t slot_stride,
+                   const int* tiles, int num_tiles, const int* runs, const int* slots, int taps, int hidden,
+                   hipStream_t stream);
+int pae_norm_join_conv_supported(int hidden);
+int pae_norm_join_conv(int dtype, float* residual, const void* y, int parts, int64_t part_stride, const void* weight,
+                       int w_is_f32, float eps, float scale, const float* filters, float* ring, int64_t slot_stride,
+                       const int* positions, const int* slots, int taps, void* rows, int num_rows, int hidden,
+                       hipStream_t stream);
 // a learned row per position added to the embedding; a layer's columns of a second token table: see token_inputs.hip
 int pae_embedding_positions(int dtype, float* out, const void* table, const int* ids, const void* rows,
                             const int* positions, int num_tokens, int hidden, int vocab, float scale, hipStream_t stream);

@@ -22,7 +22,8 @@
 // And four more, for designs that have them: a mask in chunks (`chunked`: the `window` is then a
 // chunk length, and position p sees the keys from p - p % window on, chunk borders at multiples of the length from the first token
 // of the sequence); a bias by distance, score -= slopes[head] * (p - key) (slopes null: none); a gate
-// on the output, out *= sigmoid(gate[token][head][feature]) (gate null: none); and values that are
+// on the output, out *= sigmoid(gate[token][head][feature]), or with one number a head, gate[token][head]
+// (`gate_per_head`) (gate null: none); and values that are
 // the first `vd` features of the key rows themselves (`shared_kv`, one latent row per token that
 // serves as key and as value: v_cache is then not read).
 #include "common.h"
@@ -34,7 +35,8 @@ __global__ void paged_attention_generic_kernel(
     const T* __restrict__ k_cache, const T* __restrict__ v_cache, const int* __restrict__ positions,
     const int* __restrict__ tok_seq, const int* __restrict__ block_tables, int max_blocks, int bs,
     int nh, int nkv, int hd, int vd, float scale, int window, float cap, const float* __restrict__ sinks,
-    int chunked, const float* __restrict__ slopes, const T* __restrict__ gate, int64_t gate_stride, int shared_kv) {
+    int chunked, const float* __restrict__ slopes, const T* __restrict__ gate, int64_t gate_stride, int gate_per_head,
+    int shared_kv) {
   extern __shared__ float lds[];  // [hd] query, [64] probabilities
   float* q_lds = lds;
   float* p_lds = lds + hd;
@@ -111,7 +113,7 @@ __global__ void paged_attention_generic_kernel(
     const int d = lane + i * PAE_WAVE;
     if (d < vd) {
       float v = acc[i] * inv;
-      if (gate) v *= 1.0f / (1.0f + expf(-to_f32(gate[(int64_t)t * gate_stride + (int64_t)head * vd + d])));
+      if (gate) v *= 1.0f / (1.0f + expf(-to_f32(gate[(int64_t)t * gate_stride + (gate_per_head ? head : (int64_t)head * vd + d)])));
       o[d] = from_f32<T>(v);
     }
   }
@@ -122,7 +124,7 @@ static int launch_generic(void* out, int64_t out_stride, const void* q, int64_t 
                           const void* v_cache, const int* positions, const int* tok_seq,
                           const int* block_tables, int max_blocks, int bs, int num_tokens, int nh, int nkv,
                           int hd, int vd, float scale, int window, float cap, const float* sinks, int chunked,
-                          const float* slopes, const void* gate, int64_t gate_stride, int shared_kv,
+                          const float* slopes, const void* gate, int64_t gate_stride, int gate_per_head, int shared_kv,
                           hipStream_t stream) {
   dim3 grid(num_tokens, nh);
   const size_t lds = (size_t)(hd + PAE_WAVE) * sizeof(float);
@@ -130,7 +132,7 @@ static int launch_generic(void* out, int64_t out_stride, const void* q, int64_t 
   paged_attention_generic_kernel<T, MAXD><<<grid, PAE_WAVE, lds, stream>>>(                           \
       (T*)out, out_stride, (const T*)q, q_stride, (const T*)k_cache, (const T*)v_cache, positions,    \
       tok_seq, block_tables, max_blocks, bs, nh, nkv, hd, vd, scale, window, cap, sinks, chunked,   \
-      slopes, (const T*)gate, gate_stride, shared_kv)
+      slopes, (const T*)gate, gate_stride, gate_per_head, shared_kv)
   if (vd <= 64) PAE_LAUNCH(1);
   else if (vd <= 128) PAE_LAUNCH(2);
   else if (vd <= 192) PAE_LAUNCH(3);
@@ -146,13 +148,13 @@ extern "C" int pae_paged_attention_masked(int dtype, void* out, int64_t out_stri
                                           const int* block_tables, int max_blocks, int bs,
                                           int num_tokens, int nh, int nkv, int hd, int vd, float scale,
                                           int window, float cap, const float* sinks, int chunked,
-                                          const float* slopes, const void* gate, int64_t gate_stride, int shared_kv,
-                                          hipStream_t stream) {
+                                          const float* slopes, const void* gate, int64_t gate_stride, int gate_per_head,
+                                          int shared_kv, hipStream_t stream) {
   PAE_REQUIRE(nh > 0 && nkv > 0 && nh % nkv == 0, "attention: %d query heads over %d key/value heads", nh, nkv);
   PAE_REQUIRE(hd > 0 && hd <= 1024, "attention: head_dim %d is outside 1..1024", hd);
   PAE_REQUIRE(vd > 0 && vd <= 512, "attention: value width %d is outside 1..512", vd);
   PAE_REQUIRE(!shared_kv || (nkv == 1 && vd <= hd), "attention: values shared with the keys need one key head at least as wide");
-  PAE_REQUIRE(!gate || gate_stride >= (int64_t)nh * vd, "attention: gate row stride %lld too small", (long long)gate_stride);
+  PAE_REQUIRE(!gate || gate_stride >= (gate_per_head ? nh : (int64_t)nh * vd), "attention: gate row stride %lld too small", (long long)gate_stride);
   PAE_REQUIRE(shared_kv || v_cache, "attention: no values");
   PAE_REQUIRE(bs > 0 && max_blocks > 0, "attention: bad cache geometry bs=%d max_blocks=%d", bs, max_blocks);
   PAE_REQUIRE(window >= 0, "attention: negative window %d", window);
@@ -162,11 +164,11 @@ extern "C" int pae_paged_attention_masked(int dtype, void* out, int64_t out_stri
   if (dtype == PAE_F32)
     return launch_generic<float>(out, out_stride, q, q_stride, k_cache, v_cache, positions, tok_seq, block_tables,
                                  max_blocks, bs, num_tokens, nh, nkv, hd, vd, scale, window, cap, sinks, chunked, slopes, gate,
-                                 gate_stride, shared_kv, stream);
+                                 gate_stride, gate_per_head, shared_kv, stream);
   if (dtype == PAE_BF16)
     return launch_generic<bf16_t>(out, out_stride, q, q_stride, k_cache, v_cache, positions, tok_seq, block_tables,
                                   max_blocks, bs, num_tokens, nh, nkv, hd, vd, scale, window, cap, sinks, chunked, slopes, gate,
-                                  gate_stride, shared_kv, stream);
+                                  gate_stride, gate_per_head, shared_kv, stream);
   return pae_fail("attention: unknown dtype code %d", dtype);
 }
 
@@ -179,7 +181,7 @@ extern "C" int pae_paged_attention_capped(int dtype, void* out, int64_t out_stri
   PAE_REQUIRE(vd > 0 && vd <= 256, "attention: value width %d is outside 1..256", vd);
   return pae_paged_attention_masked(dtype, out, out_stride, q, q_stride, k_cache, v_cache, positions, tok_seq,
                                     block_tables, max_blocks, bs, num_tokens, nh, nkv, hd, vd, scale, window, cap, sinks,
-                                    0, nullptr, nullptr, 0, 0, stream);
+                                    0, nullptr, nullptr, 0, 0, 0, stream);
 }
 
 extern "C" int pae_paged_attention_generic(int dtype, void* out, int64_t out_stride, const void* q,

@@ -25,6 +25,12 @@ __device__ __forceinline__ int latent_first_visible(int pos, int window, int chu
   return pos - window + 1 > 0 ? pos - window + 1 : 0;
 }
 
+// A gate on a head's output, one number a token and head: the sums of latents are multiplied by sigmoid(gate[token][head])
+// (null: no gate), which is the same as gating the values formed from them.
+__device__ __forceinline__ float latent_gate(const bf16_t* gate, int64_t gate_stride, int tok, int head) {
+  return gate ? 1.0f / (1.0f + expf(-to_f32(gate[(int64_t)tok * gate_stride + head]))) : 1.0f;
+}
+
 // tiles[i] = (table row of the sequence, first flat token, tokens, unused); blockIdx = (tile, value slice, head group)
 template <int KD, int VS, int CT>
 __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
@@ -32,7 +38,8 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
     const bf16_t* __restrict__ latent, const bf16_t* __restrict__ latent_t, const int4* __restrict__ tiles,
     const int* __restrict__ positions, const int* __restrict__ block_tables, int max_blocks, int bs, int H, int C,
     float scale_log2, int window, int chunked, int num_splits, int split_len, float* __restrict__ part_acc,
-    float* __restrict__ part_ml, const float* __restrict__ sinks) {
+    float* __restrict__ part_ml, const float* __restrict__ sinks, const bf16_t* __restrict__ head_gate,
+    int64_t gate_stride) {
   extern __shared__ float s_buf[];  // [3 or 1][CT][VS / 4 + 2][64]
   constexpr int ROWS = VS / 4 + 2;
   const int lane = threadIdx.x % PAE_WAVE, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / PAE_WAVE);
@@ -205,7 +212,7 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
     }
     // a sink joins the denominator as exp(sink), unscaled, with no key and no value
     if (sinks) sum += exp2f(sinks[head[ct]] * LOG2E - m[ct]);
-    const float inv = 1.0f / sum;
+    const float inv = latent_gate(head_gate, gate_stride, tok[ct], head[ct]) / sum;
     bf16_t* o = out + (int64_t)tok[ct] * out_stride + (int64_t)head[ct] * C + (int64_t)slice * VS;
 #pragma unroll
     for (int t = 0; t < VS / 16; ++t) {
@@ -222,7 +229,8 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
 __global__ void latent_attn_merge_kernel(bf16_t* __restrict__ out, int64_t out_stride, const float* __restrict__ part_acc,
                                          const float* __restrict__ part_ml, const int4* __restrict__ tiles,
                                          const int* __restrict__ positions, int H, int C, int window, int chunked,
-                                         int num_splits, int split_len, const float* __restrict__ sinks) {
+                                         int num_splits, int split_len, const float* __restrict__ sinks,
+                                         const bf16_t* __restrict__ head_gate, int64_t gate_stride) {
   const int4 tile = tiles[blockIdx.x];
   const int head = blockIdx.y, tok = tile.y;
   const int pos = positions[tok];
@@ -242,7 +250,7 @@ __global__ void latent_attn_merge_kernel(bf16_t* __restrict__ out, int64_t out_s
     m = m_new;
   }
   if (sinks) l += exp2f(sinks[head] * LOG2E - m);
-  const float inv = 1.0f / l;
+  const float inv = latent_gate(head_gate, gate_stride, tok, head) / l;
   s16x4 w;
 #pragma unroll
   for (int i = 0; i < 4; ++i) w[i] = bf16_bits(a[i] * inv);
@@ -275,13 +283,14 @@ extern "C" int pae_latent_attn_bf16(void* out, int64_t out_stride, const void* q
                                     const void* latent_t, const int* tiles, int num_tiles, int ct, const int* positions,
                                     const int* block_tables, int max_blocks, int bs, int H, int kd, int C, float scale,
                                     int window, int chunked, float* part_acc, float* part_ml, const float* sinks,
-                                    hipStream_t stream) {
+                                    const void* head_gate, int64_t gate_stride, hipStream_t stream) {
   PAE_REQUIRE(pae_latent_attn_supported(kd, C, bs), "latent attention: row width %d / latent %d / page size %d are not built", kd, C,
               bs);
   PAE_REQUIRE(H > 0 && H <= 16 * 65535 && max_blocks > 0 && window >= 0, "latent attention: bad sizes H=%d max_blocks=%d window=%d",
               H, max_blocks, window);
   PAE_REQUIRE(ct == 1 || ct == 2, "latent attention: %d column tiles a workgroup (1 or 2)", ct);
   PAE_REQUIRE(out_stride >= (int64_t)H * C && q_stride >= (int64_t)H * kd, "latent attention: row strides too small");
+  PAE_REQUIRE(!head_gate || gate_stride >= H, "latent attention: gate row stride %lld too small", (long long)gate_stride);
   if (num_tiles <= 0) return 0;
   const int vs = C % 128 == 0 ? 128 : (C % 64 == 0 ? 64 : 32);
   // Single tokens: the keys are split over workgroups when the tables reach beyond one split and the caller gave room
@@ -301,7 +310,7 @@ extern "C" int pae_latent_attn_bf16(void* out, int64_t out_stride, const void* q
   latent_attn_kernel<KD, VS, CT><<<grid, 256, latent_lds_bytes(CT, VS), stream>>>(                                       \
       (bf16_t*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)latent, (const bf16_t*)latent_t,             \
       (const int4*)tiles, positions, block_tables, max_blocks, bs, H, C, scale_log2, window, chunked, num_splits,       \
-      LATENT_SPLIT, part_acc, part_ml, sinks)
+      LATENT_SPLIT, part_acc, part_ml, sinks, (const bf16_t*)head_gate, gate_stride)
 #define LAT_BY_CT(KD, VS)        \
   if (ct == 1) {                 \
     LAT_LAUNCH(KD, VS, 1);       \
@@ -337,7 +346,7 @@ extern "C" int pae_latent_attn_bf16(void* out, int64_t out_stride, const void* q
     const int threads = (C / 4 + PAE_WAVE - 1) / PAE_WAVE * PAE_WAVE;
     latent_attn_merge_kernel<<<dim3(num_tiles, H), threads, 0, stream>>>((bf16_t*)out, out_stride, part_acc, part_ml,
                                                                        (const int4*)tiles, positions, H, C, window, chunked,
-                                                                       num_splits, LATENT_SPLIT, sinks);
+                                                                       num_splits, LATENT_SPLIT, sinks, (const bf16_t*)head_gate, gate_stride);
   }
   return pae_check_launch("latent_attn");
 }

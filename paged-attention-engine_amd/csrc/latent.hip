@@ -8,7 +8,8 @@
 //     [block][offset][kv_rank + rd], features 0 .. kv_rank - 1 (and, if the caller keeps them, to the
 //     pages of transposed latents, [block][kv_rank][offset]);
 //   * rotates the first `rot` of the last rd features of `down` by the token's angles, pairs
-//     (2i, 2i + 1) if `interleaved` else (i, i + rot / 2), and writes all rd behind the latent;
+//     (2i, 2i + 1) if `interleaved` else (i, i + rot / 2), cosines and sines times `magnitude`, and writes
+//     all rd behind the latent;
 //   * rotates the last rd features of every query head likewise and writes them to
 //     q_full[t][head][kv_rank .. kv_rank + rd), where the attention kernel expects them behind the
 //     head's query folded into latent space (a product that the caller launches).
@@ -23,7 +24,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void latent_prepare_kernel(
     const T* __restrict__ proj, int64_t row_stride, T* __restrict__ q_full, int64_t qf_stride, int nh, int nope, int rd,
     int rot, int interleaved, int rank, const void* __restrict__ norm_w, int w_is_f32, float eps,
-    const float* __restrict__ cos_sin, const int* __restrict__ positions, const int* __restrict__ tok_seq,
+    const float* __restrict__ cos_sin, float magnitude, const int* __restrict__ positions, const int* __restrict__ tok_seq,
     const int* __restrict__ block_tables, int max_blocks, int bs, T* __restrict__ latent, T* __restrict__ latent_t) {
   __shared__ float scratch[4];
   const int t = blockIdx.x;
@@ -47,7 +48,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
   for (int idx = threadIdx.x; idx < (nh + 1) * half; idx += 256) {
     const int h = idx / half, i = idx % half;
     const int ia = interleaved ? 2 * i : i, ib = interleaved ? 2 * i + 1 : i + half;
-    const float c = cos_sin[((int64_t)t * half + i) * 2], s = cos_sin[((int64_t)t * half + i) * 2 + 1];
+    const float c = magnitude * cos_sin[((int64_t)t * half + i) * 2], s = magnitude * cos_sin[((int64_t)t * half + i) * 2 + 1];
     const T* src = h < nh ? row + (int64_t)h * (nope + rd) + nope : down + rank;
     T* dst = h < nh ? q_full + (int64_t)t * qf_stride + (int64_t)h * (rank + rd) + rank : cached + rank;
     const float a = to_f32(src[ia]), b = to_f32(src[ib]);
@@ -65,8 +66,8 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
 
 extern "C" int pae_latent_prepare(int dtype, const void* proj, int64_t row_stride, void* q_full, int64_t qf_stride,
                                   int num_tokens, int nh, int nope, int rd, int rot, int interleaved, int rank,
-                                  const void* norm_w, int w_is_f32, float eps, const float* cos_sin, const int* positions,
-                                  const int* tok_seq, const int* block_tables, int max_blocks, int bs, void* latent,
+                                  const void* norm_w, int w_is_f32, float eps, const float* cos_sin, float magnitude,
+                                  const int* positions, const int* tok_seq, const int* block_tables, int max_blocks, int bs, void* latent,
                                   void* latent_t, hipStream_t stream) {
   PAE_REQUIRE(nh > 0 && nope > 0 && rd >= 0 && rank > 0, "latent_prepare: bad sizes nh=%d nope=%d rd=%d rank=%d", nh, nope, rd,
               rank);
@@ -81,11 +82,11 @@ extern "C" int pae_latent_prepare(int dtype, const void* proj, int64_t row_strid
   if (dtype == PAE_F32)
     latent_prepare_kernel<float><<<num_tokens, 256, 0, stream>>>(
         (const float*)proj, row_stride, (float*)q_full, qf_stride, nh, nope, rd, rot, interleaved, rank, norm_w, w_is_f32, eps,
-        cos_sin, positions, tok_seq, block_tables, max_blocks, bs, (float*)latent, (float*)latent_t);
+        cos_sin, magnitude, positions, tok_seq, block_tables, max_blocks, bs, (float*)latent, (float*)latent_t);
   else if (dtype == PAE_BF16)
     latent_prepare_kernel<bf16_t><<<num_tokens, 256, 0, stream>>>(
         (const bf16_t*)proj, row_stride, (bf16_t*)q_full, qf_stride, nh, nope, rd, rot, interleaved, rank, norm_w, w_is_f32,
-        eps, cos_sin, positions, tok_seq, block_tables, max_blocks, bs, (bf16_t*)latent, (bf16_t*)latent_t);
+        eps, cos_sin, magnitude, positions, tok_seq, block_tables, max_blocks, bs, (bf16_t*)latent, (bf16_t*)latent_t);
   else
     return pae_fail("latent_prepare: unknown dtype code %d", dtype);
   return pae_check_launch("latent_prepare");

@@ -144,7 +144,12 @@ class Model:
             paged.append(None if borrowed else mixer.paged_spec())
             # a mixer that says so keeps state of its own at a stop that borrows its pages (the inputs of
             # convolutions on its queries, say)
-            states.append(mixer.state_spec() if not borrowed or getattr(mixer, "state_when_borrowing", False) else None)
+            kept = mixer.state_spec() if not borrowed or getattr(mixer, "state_when_borrowing", False) else None
+            # what the block keeps around its mixer (the inputs of convolutions in front of its sublayers, say)
+            own = list(getattr(self.blocks[entry.layer], "state_specs", list)())
+            if own:
+                kept = tuple(([] if kept is None else [kept] if isinstance(kept, StateSpec) else list(kept)) + own)
+            states.append(kept)
         if self.plan.pair_embedding is not None:
             # what the embedding keeps per request (the token before the next one) lives behind the last stop
             paged.append(None)
@@ -195,6 +200,9 @@ class Model:
                                        and not schedule[index + 1].add_embedding)
             stream.prepared_wanted_next = (after is not None and getattr(self.blocks[after], "takes_prepared_norm", False)
                                            and not schedule[index + 1].add_embedding)
+            stream.next_conv = None
+            if after is not None and not schedule[index + 1].add_embedding:
+                stream.next_conv = getattr(self.blocks[after], "first_conv", None)
             self.blocks[entry.layer].forward(ctx, stream)
             if self.residual_tap is not None:
                 self.residual_tap(index, stream)

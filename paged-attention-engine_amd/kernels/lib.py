@@ -73,16 +73,16 @@ def _declare(lib) -> None:
         "pae_paged_attention_generic": [I, P, L, P, L, P, P, P, P, P, I, I, I, I, I, I, F, I, P],
         "pae_paged_attention_capped": [I, P, L, P, L, P, P, P, P, P, I, I, I, I, I, I, I, F, I, F, P, P],
         "pae_qk_norm_rotate_store": [I, P, L, I, I, I, I, I, P, P, I, F, I, I, P, F, P, P, P, I, I, P, P, I, I, P],
-        "pae_paged_attention_masked": [I, P, L, P, L, P, P, P, P, P, I, I, I, I, I, I, I, F, I, F, P, I, P, P, L, I, P],
+        "pae_paged_attention_masked": [I, P, L, P, L, P, P, P, P, P, I, I, I, I, I, I, I, F, I, F, P, I, P, P, L, I, I, P],
         "pae_hyper_norm": [I, P, I, P, I, L, P, I, P, P, P, P, I, F, P, P, I, I, I, P],
         "pae_hyper_spread": [P, P, I, I, I, P],
         "pae_hyper_collapse": [P, P, I, I, I, P],
         "pae_conv_norm_store": [I, P, L, P, L, I, I, P, P, P, P, P, P, L, I, I, I, I, I, I, F, P, I, I, P, P, P],
-        "pae_latent_prepare": [I, P, L, P, L, I, I, I, I, I, I, I, P, I, F, P, P, P, P, I, I, P, P, P],
+        "pae_latent_prepare": [I, P, L, P, L, I, I, I, I, I, I, I, P, I, F, P, F, P, P, P, I, I, P, P, P],
         "pae_heads_product_few": [P, L, L, P, L, L, P, I, I, I, I, P],
         "pae_latent_attn_supported": [I, I, I],
         "pae_latent_attn_columns": [I, I],
-        "pae_latent_attn_bf16": [P, L, P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, I, I, P, P, P, P],
+        "pae_latent_attn_bf16": [P, L, P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, I, I, P, P, P, P, L, P],
         "pae_latent_attn_split": [],
         "pae_gated_act": [I, P, P, I, I, I, I, P],
         "pae_gemm_plain_batched": [I, I, P, L, L, P, L, L, P, L, P, I, I, I, I, I, P],
@@ -98,6 +98,12 @@ def _declare(lib) -> None:
         "pae_moe_route": [P, I, I, I, I, I, F, P, P, P, P],
         "pae_norm_join": [I, P, I, P, P, P, P, P, P, I, F, P, I, F, P, P, I, I, P],
         "pae_linear_attention_step": [I, P, L, P, L, P, I, F, P, L, I, I, I, P, P, I, I, I, P, L, P, I, F, P, P, P],
+        "pae_fixed_decay_chunk": [I],
+        "pae_fixed_decay_step": [I, P, L, P, L, I, I, I, P, I, P, I, P, I, P, P, I, I, I, P, L, P, I, F, P, P, P],
+        "pae_input_conv_tile_rows": [I],
+        "pae_input_conv": [I, P, P, P, P, L, P, I, P, P, I, I, P],
+        "pae_norm_join_conv_supported": [I],
+        "pae_norm_join_conv": [I, P, P, I, L, P, I, F, F, P, P, L, P, P, I, P, I, I, P],
         "pae_embedding_positions": [I, P, P, P, P, P, I, I, I, F, P],
         "pae_token_gate": [I, P, P, L, P, P, I, I, I, P],
         "pae_moe_gate_up": [I, P, P, L, P, P, P, I, I, I, I, I, P],
@@ -142,6 +148,8 @@ def _declare(lib) -> None:
     lib.pae_matrix_memory_work_floats.restype = c_int64
     lib.pae_linear_attention_work_floats.argtypes = [I, I, I, I]
     lib.pae_linear_attention_work_floats.restype = c_int64
+    lib.pae_fixed_decay_work_floats.argtypes = [I, I, I, I, I]
+    lib.pae_fixed_decay_work_floats.restype = c_int64
 
 
 def _check(code: int) -> None:
@@ -979,8 +987,10 @@ def gemm_plain_heads(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor) -> Non
 HEADS_FEW_MAX_ROWS = 16
 
 
-def heads_product(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor) -> None:
-    """out[:, h, :] = a[:, h, :] @ w[h]^T for every head h (shapes as for `gemm_plain_heads`).  bfloat16 with
+def heads_product(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor,
+                  w_kn: Optional[torch.Tensor] = None) -> None:
+    """out[:, h, :] = a[:, h, :] @ w[h]^T for every head h (shapes as for `gemm_plain_heads`); `w_kn` [B, K, N] is
+    the same weights the other way round (the platform's batched product takes them so; None: turned round here).  bfloat16 with
     more rows than the few-row kernels take goes to the platform's batched matrix product, as the plain
     products of that many rows do; bfloat16 with up to 16 rows to a kernel that streams the weights once;
     everything else to the plain product's batched entry."""
@@ -998,7 +1008,10 @@ def heads_product(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor) -> None:
         return
     if a.dtype == torch.bfloat16 and a.shape[0] > SKINNY_MAX_ROWS and _RECORDING is None:
         # [B, M, K] x [B, K, N] on strided views: no copy of the operands; the result is copied into the view
-        out.copy_(torch.bmm(a.transpose(0, 1), w.transpose(1, 2)).transpose(0, 1))
+        if w_kn is None:
+            w_kn = w.transpose(1, 2).contiguous()
+        assert w_kn.shape == (w.shape[0], w.shape[2], w.shape[1]) and w_kn.is_contiguous() and w_kn.dtype == w.dtype
+        out.copy_(torch.bmm(a.transpose(0, 1), w_kn).transpose(0, 1))
         return
     gemm_plain_heads(out, a, w)
 
@@ -1057,14 +1070,21 @@ def paged_attention_capped(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Te
         _stream()))
 
 
+def _check_head_gate(gate: torch.Tensor, q: torch.Tensor, nh: int) -> None:
+    assert gate.dim() == 2 and gate.shape[0] == q.shape[0] and gate.stride(1) == 1 and gate.shape[1] >= nh
+    assert gate.dtype == q.dtype and gate.is_cuda
+
+
 def paged_attention_masked(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: Optional[torch.Tensor],
                            positions: torch.Tensor, tok_seq: torch.Tensor, block_tables: torch.Tensor,
                            nh: int, nkv: int, hd: int, vd: int, scale: float, window: int = 0, chunked: bool = False,
                            slopes: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
-                           softcap: float = 0.0, sinks: Optional[torch.Tensor] = None) -> None:
+                           softcap: float = 0.0, sinks: Optional[torch.Tensor] = None,
+                           head_gate: Optional[torch.Tensor] = None) -> None:
     """`paged_attention_capped` with, each optional: the `window` read as a chunk length (`chunked`:
     position p sees keys from p - p % window on), a bias by distance (score -= slopes[h] * (p - key),
-    float32 [nh]), and an output gate (out *= sigmoid(gate), `gate` a [T, >= nh * vd] view of rows).
+    float32 [nh]), and an output gate (out *= sigmoid(gate), `gate` a [T, >= nh * vd] view of rows, or
+    `head_gate` a [T, >= nh] view with one number a head).
     `v_cache` None: the values are the first `vd` features of the key rows, which are then one row
     per token, `k_cache` [block][bs][hd] (nkv must be 1)."""
     _not_while_recording("paged_attention_masked")
@@ -1089,11 +1109,16 @@ def paged_attention_masked(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Te
         assert gate.dim() == 2 and gate.shape[0] == T and gate.stride(1) == 1 and gate.shape[1] >= nh * vd
         assert gate.dtype == q.dtype
         gate_stride = gate.stride(0)
+    if head_gate is not None:
+        assert gate is None
+        _check_head_gate(head_gate, q, nh)
+        gate, gate_stride = head_gate, head_gate.stride(0)
     _check(library().pae_paged_attention_masked(
         code_of(q.dtype), out.data_ptr(), out.stride(0), q.data_ptr(), q.stride(0), k_cache.data_ptr(),
         _ptr(v_cache), positions.data_ptr(), tok_seq.data_ptr(), block_tables.data_ptr(),
         block_tables.shape[1], bs, T, nh, nkv, hd, vd, float(scale), int(window), float(softcap), _ptr(sinks),
-        1 if chunked else 0, _ptr(slopes), _ptr(gate), gate_stride, 1 if v_cache is None else 0, _stream()))
+        1 if chunked else 0, _ptr(slopes), _ptr(gate), gate_stride, 1 if head_gate is not None else 0,
+        1 if v_cache is None else 0, _stream()))
 
 
 def conv_norm_store(proj: torch.Tensor, q_out: torch.Tensor, tok_seq: torch.Tensor, positions: torch.Tensor,
@@ -1142,10 +1167,10 @@ def conv_norm_store(proj: torch.Tensor, q_out: torch.Tensor, tok_seq: torch.Tens
 def latent_prepare(proj: torch.Tensor, q_full: torch.Tensor, nh: int, nope: int, rd: int, rot: int, interleaved: bool,
                    rank: int, norm_w: torch.Tensor, eps: float, cos_sin: Optional[torch.Tensor], positions: torch.Tensor,
                    tok_seq: torch.Tensor, block_tables: torch.Tensor, latent: torch.Tensor,
-                   latent_t: Optional[torch.Tensor] = None) -> None:
+                   latent_t: Optional[torch.Tensor] = None, magnitude: float = 1.0) -> None:
     """Rows `proj` [T, nh (nope + rd) + rank + rd] = [query heads | down projection]: the first `rank`
     features of the down projection are RMS-normed with `norm_w` and, with the last rd (their first
-    `rot` rotated by `cos_sin`), written to the token's row of `latent` [block][bs][rank + rd]; the
+    `rot` rotated by `cos_sin` times `magnitude`), written to the token's row of `latent` [block][bs][rank + rd]; the
     query heads' last rd features are rotated likewise into q_full[t, h, rank:] (`q_full`
     [T, nh * (rank + rd)], whose first `rank` features per head the caller fills).  With `latent_t`
     [block][rank][bs] the normed latents are also written transposed within the page."""
@@ -1166,8 +1191,8 @@ def latent_prepare(proj: torch.Tensor, q_full: torch.Tensor, nh: int, nope: int,
     wp, wf = _param(norm_w)
     _check(library().pae_latent_prepare(
         code_of(proj.dtype), proj.data_ptr(), proj.stride(0), q_full.data_ptr(), q_full.stride(0), T, nh, nope, rd, rot,
-        1 if interleaved else 0, rank, wp, wf, float(eps), _ptr(cos_sin) if rot else None, positions.data_ptr(),
-        tok_seq.data_ptr(), block_tables.data_ptr(), block_tables.shape[1], latent.shape[1], latent.data_ptr(),
+        1 if interleaved else 0, rank, wp, wf, float(eps), _ptr(cos_sin) if rot else None, float(magnitude),
+        positions.data_ptr(), tok_seq.data_ptr(), block_tables.data_ptr(), block_tables.shape[1], latent.shape[1], latent.data_ptr(),
         _ptr(latent_t), _stream()))
 
 
@@ -1183,16 +1208,20 @@ def latent_attn_tokens(num_heads: int, column_tiles: int) -> int:
 
 def latent_attn(out: torch.Tensor, q_full: torch.Tensor, latent: torch.Tensor, latent_t: torch.Tensor, tiles: torch.Tensor,
                 column_tiles: int, positions: torch.Tensor, block_tables: torch.Tensor, nh: int, rank: int, scale: float,
-                window: int = 0, chunked: bool = False, sinks: Optional[torch.Tensor] = None) -> None:
+                window: int = 0, chunked: bool = False, sinks: Optional[torch.Tensor] = None,
+                head_gate: Optional[torch.Tensor] = None) -> None:
     """Latent attention on the matrix cores.  `q_full` [T, nh * KD] holds per head the query folded into
     latent space and its rotated part; `latent` [block][bs][KD] and `latent_t` [block][rank][bs] are the
     cached rows and their transposed latents; tiles[i] = (table row, first flat token, tokens, 0) with at
     most `latent_attn_tokens(nh, column_tiles)` tokens; out[t, h * rank:(h + 1) * rank] receives the
-    weighted sums of the latents.  `sinks` float32 [nh]: exp(sink) joins each head's denominator."""
+    weighted sums of the latents.  `sinks` float32 [nh]: exp(sink) joins each head's denominator.  `head_gate`
+    [T, >= nh] (a view of wider rows will do): a head's sums are multiplied by sigmoid of its number."""
     _not_while_recording("latent_attn")
     _gpu(out, q_full, latent, latent_t, tiles, positions, block_tables, sinks)
     if sinks is not None:
         assert sinks.dtype == torch.float32 and sinks.numel() == nh and sinks.is_contiguous()
+    if head_gate is not None:
+        _check_head_gate(head_gate, q_full, nh)
     T = q_full.shape[0]
     kd, bs = latent.shape[2], latent.shape[1]
     assert q_full.dtype == torch.bfloat16 == out.dtype == latent.dtype == latent_t.dtype
@@ -1213,7 +1242,7 @@ def latent_attn(out: torch.Tensor, q_full: torch.Tensor, latent: torch.Tensor, l
         out.data_ptr(), out.stride(0), q_full.data_ptr(), q_full.stride(0), latent.data_ptr(), latent_t.data_ptr(),
         tiles.data_ptr(), tiles.shape[0], column_tiles, positions.data_ptr(), block_tables.data_ptr(), block_tables.shape[1],
         bs, nh, kd, rank, float(scale), int(window), 1 if chunked else 0, _ptr(part_acc), _ptr(part_ml), _ptr(sinks),
-        _stream()))
+        _ptr(head_gate), head_gate.stride(0) if head_gate is not None else 0, _stream()))
 
 
 def hyper_norm(streams: torch.Tensor, num_streams: int, y: Optional[torch.Tensor], layer_scale: Optional[torch.Tensor],
@@ -1587,6 +1616,117 @@ def linear_attention_step(proj: torch.Tensor, decay_in: torch.Tensor, decay_bias
         gate.data_ptr(), gate.stride(0), 1 if gate_activation == "sigmoid" else 0, T, S, seq_runs.data_ptr(),
         slots.data_ptr(), H, D, V, state.data_ptr(), state.stride(0), wp, wf, float(norm_eps), work.data_ptr(),
         out.data_ptr(), _stream()))
+
+
+def fixed_decay_chunk(key_dim: int) -> int:
+    """Tokens a chunk of `fixed_decay_step` holds for that key width; 0: its runs of any length go token by token."""
+    return library().pae_fixed_decay_chunk(int(key_dim))
+
+
+def fixed_decay_step(proj: torch.Tensor, gate: torch.Tensor, out: torch.Tensor, serial: torch.Tensor, chunks: torch.Tensor,
+                     scans: torch.Tensor, slots: torch.Tensor, powers: torch.Tensor, state: torch.Tensor,
+                     norm_w: torch.Tensor, H: int, D: int, V: int, norm_eps: float, silu: bool = True,
+                     gate_activation: str = "sigmoid") -> None:
+    """Linear attention with a fixed decay per head over a step's rows.  `proj` [T, >= 2HD + HV] holds per token
+    [q | k | v] before the activation (SiLU, or none with `silu` False); `gate` [T, HV] is a view of rows in proj's
+    type.  The step's runs of tokens are in three int32 lists of rows of four: `serial` (table row, first flat row,
+    rows, 0) for those walked token by token; `chunks` likewise for the pieces of the others, up to
+    `fixed_decay_chunk(D)` rows each and in order; `scans` (table row, first chunk, chunks, rows of the last chunk) per
+    run in pieces.  `slots` int32 [S]; `powers` float32 [H, chunk + 1] holds every head's decay to the powers 0 .. chunk
+    (2 columns where there are no chunks); `state` float32 [slots, H, V, D] is read and moved on; `out` [T, H * V]
+    receives the read-out, normed over the whole row with `norm_w` [H * V] and gated, in proj's type."""
+    _not_while_recording("fixed_decay_step")
+    _gpu(proj, gate, out, serial, chunks, scans, slots, powers, state, norm_w)
+    T = proj.shape[0]
+    assert gate_activation in ("silu", "sigmoid")
+    assert proj.dim() == 2 and proj.stride(1) == 1 and proj.shape[1] >= 2 * H * D + H * V
+    assert gate.dim() == 2 and gate.shape == (T, H * V) and gate.dtype == proj.dtype and gate.stride(1) == 1
+    assert out.shape == (T, H * V) and out.is_contiguous() and out.dtype == proj.dtype
+    for lists in (serial, chunks, scans):
+        assert lists.dtype == torch.int32 and lists.dim() == 2 and lists.shape[1] == 4 and lists.is_contiguous()
+        assert lists.numel() == 0 or lists.data_ptr() % 16 == 0
+    assert slots.dtype == torch.int32 and slots.is_contiguous()
+    assert powers.dtype == torch.float32 and powers.shape == (H, (fixed_decay_chunk(D) or 1) + 1) and powers.is_contiguous()
+    assert state.dtype == torch.float32 and tuple(state.shape[1:]) == (H, V, D) and state[0].is_contiguous()
+    assert norm_w.numel() == H * V and norm_w.is_contiguous()
+    wp, wf = _param(norm_w)
+    lib = library()
+    work = torch.empty(lib.pae_fixed_decay_work_floats(T, chunks.shape[0], H, D, V), dtype=torch.float32, device=proj.device)
+    _check(lib.pae_fixed_decay_step(
+        code_of(proj.dtype), proj.data_ptr(), proj.stride(0), gate.data_ptr(), gate.stride(0),
+        1 if gate_activation == "sigmoid" else 0, 1 if silu else 0, T, serial.data_ptr(), serial.shape[0], chunks.data_ptr(),
+        chunks.shape[0], scans.data_ptr(), scans.shape[0], slots.data_ptr(), powers.data_ptr(), H, D, V, state.data_ptr(),
+        state.stride(0), wp, wf, float(norm_eps), work.data_ptr(), out.data_ptr(), _stream()))
+
+
+def input_conv_tile_rows(taps: int) -> int:
+    """Rows of a sequence that one tile of `input_conv` takes at most."""
+    return library().pae_input_conv_tile_rows(int(taps))
+
+
+def _check_ring(ring: Optional[torch.Tensor], filters: torch.Tensor, hidden: int) -> int:
+    """The slot stride of a convolution's state [slots, taps - 1, hidden] (None with one tap: it keeps nothing)."""
+    taps = filters.shape[0]
+    assert filters.dtype == torch.float32 and filters.shape == (taps, hidden) and filters.is_contiguous()
+    if taps == 1:
+        return 0
+    assert ring is not None and ring.dtype == torch.float32 and tuple(ring.shape[1:]) == (taps - 1, hidden)
+    assert ring[0].is_contiguous()
+    return ring.stride(0)
+
+
+def input_conv(residual: torch.Tensor, dtype: torch.dtype, filters: torch.Tensor, ring: Optional[torch.Tensor],
+               tiles: torch.Tensor, seq_runs: torch.Tensor, slots: torch.Tensor) -> torch.Tensor:
+    """[T, H] in `dtype`: the float32 stream plus a causal convolution of it over each sequence's own tokens.
+    `filters` float32 [taps, H], the last tap the token's own; `ring` float32 [slots, taps - 1, H] holds a request's
+    last inputs, the one at position p in row p % (taps - 1), and is moved on.  `tiles` int32 [n, 4] = (table row of
+    the sequence, first flat row, rows, rows of the sequence in this step before the tile), up to
+    `input_conv_tile_rows(taps)` rows each; `seq_runs` int32 [S, 4] = (first row, rows, tokens before, 0)."""
+    _not_while_recording("input_conv")
+    _gpu(residual, filters, ring, tiles, seq_runs, slots)
+    T, H = residual.shape
+    assert residual.dtype == torch.float32 and residual.is_contiguous()
+    for lists in (tiles, seq_runs):
+        assert lists.dtype == torch.int32 and lists.dim() == 2 and lists.shape[1] == 4 and lists.is_contiguous()
+        assert lists.data_ptr() % 16 == 0
+    assert slots.dtype == torch.int32 and slots.numel() >= seq_runs.shape[0] and slots.is_contiguous()
+    stride = _check_ring(ring, filters, H)
+    out = torch.empty((T, H), dtype=dtype, device=residual.device)
+    _check(library().pae_input_conv(code_of(dtype), out.data_ptr(), residual.data_ptr(), filters.data_ptr(), _ptr(ring), stride,
+                                    tiles.data_ptr(), tiles.shape[0], seq_runs.data_ptr(), slots.data_ptr(), filters.shape[0],
+                                    H, _stream()))
+    return out
+
+
+def norm_join_conv_supported(hidden: int) -> bool:
+    return bool(library().pae_norm_join_conv_supported(int(hidden)))
+
+
+def norm_join_conv(residual: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, scale: float,
+                   dtype: torch.dtype, filters: torch.Tensor, ring: Optional[torch.Tensor], positions: torch.Tensor,
+                   slots: torch.Tensor) -> torch.Tensor:
+    """For a step in which row t is the one token of sequence t: `norm_scale_add` of `y` and `input_conv` of the new
+    stream in one kernel.  Returns the convolution's rows in `dtype`; the stream and the ring are moved on."""
+    _not_while_recording("norm_join_conv")
+    _gpu(residual, y, weight, filters, ring, positions, slots)
+    T, H = residual.shape
+    assert residual.dtype == torch.float32 and residual.is_contiguous() and y.is_contiguous()
+    parts = 0
+    if y.dim() == 3:
+        assert y.dtype == torch.float32 and tuple(y.shape[1:]) == (T, H)
+        parts = y.shape[0]
+    else:
+        assert tuple(y.shape) == (T, H) and y.dtype == dtype
+    assert weight.numel() == H
+    for t in (positions, slots):
+        assert t.dtype == torch.int32 and t.numel() >= T and t.is_contiguous()
+    stride = _check_ring(ring, filters, H)
+    out = torch.empty((T, H), dtype=dtype, device=residual.device)
+    wp, wf = _param(weight)
+    _check(library().pae_norm_join_conv(code_of(dtype), residual.data_ptr(), y.data_ptr(), parts, T * H, wp, wf, float(eps),
+                                        float(scale), filters.data_ptr(), _ptr(ring), stride, positions.data_ptr(),
+                                        slots.data_ptr(), filters.shape[0], out.data_ptr(), T, H, _stream()))
+    return out
 
 
 def project_f32(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None) -> torch.Tensor:

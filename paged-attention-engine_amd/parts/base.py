@@ -95,9 +95,11 @@ class ResidualStream:
         self.sum_weights: Optional[torch.Tensor] = None
         # for blocks that hand the next block its first norm's rows: (that norm, the whole stream normed by it),
         # left by the kernel that last wrote the stream, and whether the block after this one will take them
-        # (set by the model)
+        # (set by the model); likewise (a convolution, its rows) for blocks that read the stream through one, with
+        # the convolution in front of the block after this one in `next_conv` (set by the model)
         self.prepared: Optional[tuple] = None
         self.prepared_wanted_next = False
+        self.next_conv: Optional[object] = None
 
 
 class BranchTerms(list):

@@ -9,6 +9,7 @@ from __future__ import annotations
 
 from .base import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, BranchSink, BranchTerms, Part, ResidualStream, ScaleShape,
                    StreamJoin, build_part, plain_rows, register_block)
+from .input_conv import InputConv
 
 
 @register_block("prenorm")
@@ -79,9 +80,12 @@ class BranchNormBlock:
     x <- x + m * norm1(mixer(x)); x <- x + m * norm2(feed_forward(x)), m = `residual_scale`.
     A layer whose spec names no feed-forward has the first half only.  The stream is float32; a
     branch's product reads it rounded to the activation type, which the kernel that adds a branch
-    writes on the way for the branch after it (`stream.rows`)."""
+    writes on the way for the branch after it (`stream.rows`).
 
-    reads_stream_rows = True
+    With `input_conv` in the spec the branches read the stream through a convolution over time, c(x) instead of x
+    (see parts/input_conv.py), with state of the block's own per request.  In a step of single tokens one kernel
+    joins a branch and forms the rows of the convolution after it, also of the next block's first
+    (`stream.next_conv`, handed on as `stream.prepared`)."""
 
     def __init__(self, layer_spec, dtype, device):
         self.spec = layer_spec
@@ -95,6 +99,25 @@ class BranchNormBlock:
         for norm in (self.mixer_out_norm, self.feed_forward_out_norm):
             if norm is not None and not hasattr(norm, "add_scaled"):
                 raise ValueError(f"the norm '{norm.spec.kind}' cannot stand on a branch's output (no add_scaled)")
+        self.mixer_conv = self.feed_forward_conv = None
+        if layer_spec.input_conv is not None:
+            width = layer_spec.mixer_norm.size
+            self.mixer_conv = InputConv(layer_spec.input_conv, 0, width, dtype, device)
+            if self.feed_forward is not None:
+                self.feed_forward_conv = InputConv(layer_spec.input_conv, 1, width, dtype, device)
+
+    @property
+    def reads_stream_rows(self) -> bool:
+        return self.mixer_conv is None
+
+    @property
+    def first_conv(self):
+        return self.mixer_conv
+
+    def state_specs(self):
+        """What the block itself keeps per request, beside its mixer."""
+        convs = [conv.state_spec() for conv in (self.mixer_conv, self.feed_forward_conv) if conv is not None]
+        return [spec for spec in convs if spec is not None]
 
     def _named(self):
         s = self.spec
@@ -102,6 +125,7 @@ class BranchNormBlock:
         if self.feed_forward is not None:
             out += [(self.feed_forward_out_norm, s.prefix + s.feed_forward_norm_prefix),
                     (self.feed_forward, s.prefix + s.feed_forward_prefix)]
+        out += [(conv, s.prefix) for conv in (self.mixer_conv, self.feed_forward_conv) if conv is not None]
         return out
 
     @property
@@ -145,6 +169,8 @@ class BranchNormBlock:
         if stream.pending is not None or stream.owed is not None:
             raise ValueError("a block with its norms on the branches' outputs follows one that left a branch pending")
         ctx.sink = None
+        if self.mixer_conv is not None:
+            return self._forward_convolved(ctx, stream)
         has_ff = self.feed_forward is not None
         y = self.mixer.forward(ctx, self._rows(stream))
         # the rows of the new stream are wanted by this block's feed-forward, or by a block of this
@@ -154,6 +180,33 @@ class BranchNormBlock:
         if has_ff:
             y = self.feed_forward.forward(ctx, self._rows(stream))
             self._join(stream, self.feed_forward_out_norm, y, follows)
+
+    def _forward_convolved(self, ctx, stream: ResidualStream) -> None:
+        entry, nxt = ctx.entry, stream.next_conv
+        prepared, stream.prepared = stream.prepared, None
+        if prepared is not None and prepared[0] is self.mixer_conv:
+            x = prepared[1]
+        else:
+            x = self.mixer_conv.forward(ctx, stream.residual, entry)
+        y = self.mixer.forward(ctx, x)
+        if self.feed_forward is not None:
+            x = self._join_and_convolve(ctx, stream, self.mixer_out_norm, y, self.feed_forward_conv, entry)
+            if x is None:
+                x = self.feed_forward_conv.forward(ctx, stream.residual, entry)
+            y = self.feed_forward.forward(ctx, x)
+        norm = self.mixer_out_norm if self.feed_forward is None else self.feed_forward_out_norm
+        x = self._join_and_convolve(ctx, stream, norm, y, nxt, entry + 1)
+        if x is not None:
+            stream.prepared = (nxt, x)
+
+    def _join_and_convolve(self, ctx, stream: ResidualStream, norm, y, conv, entry: int):
+        """x <- x + m * norm(y).  In a step of single tokens also the rows of the convolution `conv` that reads the
+        stream next, at stop `entry`; else None (the reader runs a kernel of its own)."""
+        from ..kernels import lib as K
+        if conv is not None and ctx.num_tokens == ctx.num_seqs and K.norm_join_conv_supported(stream.residual.shape[1]):
+            return conv.join_and_forward(ctx, stream.residual, y, norm, self.spec.residual_scale, entry)
+        norm.add_scaled(stream.residual, y, self.spec.residual_scale)
+        return None
 
 
 @register_block("hyper")

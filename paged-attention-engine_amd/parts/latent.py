@@ -7,13 +7,14 @@ value W_uv_j c; query and shared key part are rotated by position; the score is
 
     (q_nope . W_uk_j c + q_rot . k_rot) * scale
 
-over the keys the mask lets through (a sliding window, chunks, or every earlier key), an ordinary
+(cosines and sines times the position encoding's magnitude, if it has one) over the keys the mask lets through (a sliding window, chunks, or every earlier key), an ordinary
 softmax, and W_o on the concatenated heads.
 
 For designs that have them: a learned sink per head that joins the softmax's denominator as exp(sink), without
 a key or a value and not scaled (`sinks`); no rotated part at all (`rope_dim` 0); and layers without a down
 projection that read the rows an earlier layer cached, with their own W_uk, W_uv, queries and mask (`own_kv` False:
-the stop borrows that layer's pages).
+the stop borrows that layer's pages); a gate on every head's output, sigmoid of one number per token and head, a
+projection of the mixer's input (`gate_name`): applied to the head's sum of latents, which W_uv_j then takes over.
 
 What the cache holds of a token is c and the rotated part, one row of kv_rank + rope_dim whatever the number
 of heads (`paged_spec`: one tensor "latent" [PAGE][kv_rank + rope_dim]).  The heads' keys and values
@@ -21,7 +22,7 @@ are never formed: since q_nope . (W_uk_j c) = (W_uk_j^T q_nope) . c, the query i
 space once per token ([W_uk_j^T q_nope | q_rot], kv_rank + rope_dim wide), the attention kernel scores
 it against the cached row as it is and sums the rows' first kv_rank features as values, and the
 head's output is W_uv_j times that sum.  The query projection and the down projection are one
-product; the two per-head products are one launch each.
+product (a gate's rows ride in it); the two per-head products are one launch each.
 """
 
 from __future__ import annotations
@@ -77,8 +78,8 @@ class LatentAttention(Part):
             raise ValueError(f"{rotated} rotated features of a rotated part of {spec.rope_dim}")
         self.position = (build_part(POSITION_ENCODINGS, "position encoding", spec.position, dtype, device)
                          if spec.position is not None else POSITION_ENCODINGS["none"](None, dtype, device))
-        if not hasattr(self.position, "rotary_table") or float(getattr(self.position, "magnitude", 1.0)) != 1.0:
-            raise ValueError("latent attention rotates by a plain table of cosines and sines")
+        if not hasattr(self.position, "rotary_table"):
+            raise ValueError("latent attention rotates by a table of cosines and sines")
 
     @property
     def graph_safe(self) -> bool:
@@ -124,12 +125,19 @@ class LatentAttention(Part):
             out[prefix + s.down_norm_name] = ScaleShape((s.kv_rank,))
         if s.sinks:
             out[prefix + s.sink_name] = (s.num_heads,)
+        if s.gate_name is not None:
+            out[prefix + s.gate_name + sfx] = (s.num_heads, s.hidden_size)
         return out
 
     def bind(self, prefix, weights):
         s = self.spec
         sfx = s.weight_suffix
         projected = [weights[prefix + s.q_name + sfx]] + ([weights[prefix + s.down_name + sfx]] if s.own_kv else [])
+        if s.gate_name is not None:
+            projected.append(weights[prefix + s.gate_name + sfx])
+            rows = sum(w.shape[0] for w in projected)
+            if rows % 8:  # rows of zeros: the product's rows then start on 16-byte boundaries
+                projected.append(torch.zeros((8 - rows % 8, s.hidden_size), dtype=projected[0].dtype, device=projected[0].device))
         self.proj = Linear(self.matrix(torch.cat(projected, dim=0)))
         self.down_norm = self.vector(weights[prefix + s.down_norm_name]) if s.own_kv else None
         # sinks enter the softmax, which is float32
@@ -139,6 +147,10 @@ class LatentAttention(Part):
         # the fold q_nope -> W_uk^T q_nope is a product with W_uk^T as its [out, in] matrix, head by head
         self.up_k_t = self.matrix(up_k.transpose(1, 2))
         self.up_v = self.matrix(weights[prefix + s.up_v_name + sfx].view(s.num_heads, s.value_dim, s.kv_rank))
+        # both the other way round as well, for steps of many rows (see kernels.lib.heads_product)
+        self.up_k = self.up_v_t = None
+        if self.dtype == torch.bfloat16:
+            self.up_k, self.up_v_t = self.matrix(up_k), self.matrix(self.up_v.transpose(1, 2))
         self.out = Linear(self.matrix(weights[prefix + s.o_name + sfx]))
 
     def forward(self, ctx, x):
@@ -151,12 +163,17 @@ class LatentAttention(Part):
         latent, latent_t = pages["latent"], pages.get("latent_t")
         table = ctx.block_tables[ctx.cache.group_of(ctx.cache_entry)]
         proj = self.proj(x)
+        gate = None
+        if s.gate_name is not None:
+            first = H * (D + R) + (C + R if s.own_kv else 0)
+            gate = proj[:, first:first + H]
         rot, cos_sin = self.position.rotary_table(ctx)
         q_full = torch.empty((T, H * (C + R)), dtype=proj.dtype, device=proj.device)
         if s.own_kv:
             K.latent_prepare(proj, q_full, H, D, R, rot, bool(getattr(self.position, "interleaved", False)), C,
-                             self.down_norm, s.norm_eps, cos_sin, ctx.positions, ctx.tok_seq, table, latent, latent_t)
-        K.heads_product(q_full.view(T, H, C + R)[:, :, :C], proj[:, :H * (D + R)].view(T, H, D + R)[:, :, :D], self.up_k_t)
+                             self.down_norm, s.norm_eps, cos_sin, ctx.positions, ctx.tok_seq, table, latent, latent_t,
+                             magnitude=float(getattr(self.position, "magnitude", 1.0)))
+        K.heads_product(q_full.view(T, H, C + R)[:, :, :C], proj[:, :H * (D + R)].view(T, H, D + R)[:, :, :D], self.up_k_t, self.up_k)
         summed = torch.empty((T, H * C), dtype=proj.dtype, device=proj.device)
         key = self.step_lists_key(ctx.cache.block_size)
         if key is not None and latent_t is not None:
@@ -164,10 +181,10 @@ class LatentAttention(Part):
             for name, column_tiles in (("single", 1), ("runs", 2)):
                 if tiles[name].numel():
                     K.latent_attn(summed, q_full, latent, latent_t, tiles[name], column_tiles, ctx.positions, table, H, C,
-                                  s.scale, s.window or 0, s.mask == "chunk", self.sinks)
+                                  s.scale, s.window or 0, s.mask == "chunk", self.sinks, head_gate=gate)
         else:
             K.paged_attention_masked(summed, q_full, latent, None, ctx.positions, ctx.tok_seq, table, H, 1, C + R, C, s.scale,
-                                     s.window or 0, s.mask == "chunk", sinks=self.sinks)
+                                     s.window or 0, s.mask == "chunk", sinks=self.sinks, head_gate=gate)
         heads = torch.empty((T, H * V), dtype=proj.dtype, device=proj.device)
-        K.heads_product(heads.view(T, H, V), summed.view(T, H, C), self.up_v)
+        K.heads_product(heads.view(T, H, V), summed.view(T, H, C), self.up_v, self.up_v_t)
         return self.out.branch(heads, ctx.sink)

@@ -1,4 +1,7 @@
-"""Gated linear attention: a recurrent mixer that keeps, per request, one matrix per head that decays by a
+"""Linear attention with a decaying state: with a learned decay per token and key channel
+(`GatedLinearAttention`), and with a fixed decay per head (`FixedDecayAttention`, below).
+
+Gated linear attention: a recurrent mixer that keeps, per request, one matrix per head that decays by a
 learned factor per key channel, instead of keys and values per token.
 
 Per token, with h the mixer's input:  q = W_q h * D^-1/2 and k = W_k h (H heads of D), v = W_v h (H heads of V);
@@ -105,10 +108,107 @@ class GatedLinearAttention(Part):
         proj = self.proj(x)
         gate = proj[:, 2 * H * D + H * V:2 * H * D + 2 * H * V]
         decay_in = self.decay_up(proj[:, self.narrow_at:self.narrow_at + self.narrow_width])
-        state = ctx.cache.state_of(ctx.cache_entry)
-        if isinstance(state, dict):  # beside another mixer that keeps state, the tensors are found by name
-            state = state["matrices"]
+        state = ctx.cache.state_of(ctx.cache_entry, "matrices")
         out = torch.empty((x.shape[0], H * V), dtype=x.dtype, device=x.device)
         K.linear_attention_step(proj, decay_in, self.decay_bias, s.decay_temperature, gate, out, ctx.memo[SEQ_RUNS]["runs"],
                                 ctx.slots, state, self.norm, H, D, V, s.norm_eps, s.gate_activation)
+        return self.out.branch(out, ctx.sink)
+
+
+SERIAL_ROWS = 16  # runs of up to this many tokens walk the recurrence token by token, longer ones go in chunks
+
+
+def decay_runs(shape: StepShape, chunk: int):
+    """Work lists of `kernels.lib.fixed_decay_step` for chunks of `chunk` tokens (0: no chunks)."""
+    serial, chunks, scans = [], [], []
+    for row, (start, n) in enumerate(zip(shape.q_starts, shape.q_lens)):
+        if n <= SERIAL_ROWS or not chunk:
+            serial += [row, start, n, 0]
+            continue
+        first = len(chunks) // 4
+        for at in range(0, n, chunk):
+            chunks += [row, start + at, min(chunk, n - at), 0]
+        scans += [row, first, len(chunks) // 4 - first, n - (n - 1) // chunk * chunk]
+    return {"serial": (serial, 4), "chunks": (chunks, 4), "scans": (scans, 4)}
+
+
+@register_mixer("fixed_decay_linear_attention")
+class FixedDecayAttention(Part):
+    """Lightning attention: per token q = act(W_q h) and k = act(W_k h) (H heads of D), v = act(W_v h) (H heads of V),
+    act = SiLU or none by the spec; head j moves its state on by S <- a_j S + k v^T with a fixed decay a_j and reads
+    o = S^T q.  All heads' o are divided by their common root mean square over H V, multiplied by a weight [H V] and
+    by sigmoid(W_g h) (or SiLU), and projected out by W_o.
+
+    The projections that read h are one product.  The state is a float32 tensor "matrices" [H, V, D] per request,
+    zeroed when a request takes the slot.  Everything after the projections is float32 inside
+    `kernels.lib.fixed_decay_step`, which takes short runs token by token and longer ones in chunks."""
+
+    graph_safe = True
+
+    def __init__(self, spec, dtype, device):
+        super().__init__(spec, dtype, device)
+        if min(spec.num_heads, spec.key_dim, spec.value_dim) <= 0:
+            raise ValueError("linear attention with fixed decays: heads, key_dim and value_dim must be positive")
+        if spec.key_dim > 1024:
+            raise ValueError(f"linear attention with fixed decays: key_dim {spec.key_dim}: the kernels take up to 1024")
+        if len(spec.decays) != spec.num_heads:
+            raise ValueError(f"{len(spec.decays)} decays for {spec.num_heads} heads")
+        if spec.activation not in ("silu", "none"):
+            raise ValueError(f"activation '{spec.activation}' is not known (known: silu, none)")
+        if spec.gate_activation not in ("silu", "sigmoid"):
+            raise ValueError(f"gate_activation '{spec.gate_activation}' is not known (known: silu, sigmoid)")
+
+    @property
+    def graph_max_rows(self):
+        s = self.spec
+        return rows_a_graph_may_hold(self.dtype, s.hidden_size, s.num_heads * s.value_dim)
+
+    def state_spec(self):
+        s = self.spec
+        return StateSpec((s.num_heads, s.value_dim, s.key_dim), torch.float32, "matrices")
+
+    @property
+    def chunk(self) -> int:
+        return K.fixed_decay_chunk(self.spec.key_dim)
+
+    def step_lists_key(self, block_size: int):
+        return ("runs under a fixed decay", self.chunk)
+
+    def step_lists(self, shape: StepShape):
+        return decay_runs(shape, self.chunk)
+
+    def _projections(self):
+        s = self.spec
+        hd, hv = s.num_heads * s.key_dim, s.num_heads * s.value_dim
+        return ((s.q_name, hd), (s.k_name, hd), (s.v_name, hv), (s.gate_name, hv))
+
+    def tensors(self, prefix):
+        s = self.spec
+        out = {prefix + name + s.weight_suffix: (rows, s.hidden_size) for name, rows in self._projections()}
+        out[prefix + s.norm_name] = ScaleShape((s.num_heads * s.value_dim,))
+        out[prefix + s.o_name + s.weight_suffix] = (s.hidden_size, s.num_heads * s.value_dim)
+        return out
+
+    def bind(self, prefix, weights):
+        s = self.spec
+        self.proj = Linear(self.matrix(torch.cat([weights[prefix + name + s.weight_suffix] for name, _ in self._projections()], dim=0)))
+        self.norm = self.vector(weights[prefix + s.norm_name])
+        self.out = Linear(self.matrix(weights[prefix + s.o_name + s.weight_suffix]))
+        # powers of the decays, formed in float64 and rounded once
+        exponents = torch.arange((self.chunk or 1) + 1, dtype=torch.float64)
+        self.powers = torch.pow(torch.tensor(s.decays, dtype=torch.float64)[:, None], exponents).to(
+            device=self.device, dtype=torch.float32).contiguous()
+
+    def forward(self, ctx, x):
+        s = self.spec
+        if not ctx.writes_cache:
+            raise ValueError("a recurrent mixer cannot borrow another stop's state")
+        x = plain_rows(x)
+        H, D, V = s.num_heads, s.key_dim, s.value_dim
+        proj = self.proj(x)
+        lists = ctx.memo[self.step_lists_key(ctx.cache.block_size)]
+        out = torch.empty((x.shape[0], H * V), dtype=x.dtype, device=x.device)
+        K.fixed_decay_step(proj, proj[:, 2 * H * D + H * V:], out, lists["serial"], lists["chunks"], lists["scans"], ctx.slots,
+                           self.powers, ctx.cache.state_of(ctx.cache_entry, "matrices"), self.norm, H, D, V, s.norm_eps,
+                           s.activation == "silu", s.gate_activation)
         return self.out.branch(out, ctx.sink)

@@ -21,7 +21,7 @@ class RMSNorm(Part):
     graph_safe = True
     def tensors(self, prefix):
         # a weight that is stored minus an offset lies around zero like any other tensor
-        shape = (self.spec.size,)
+        shape = () if self.spec.one_weight else (self.spec.size,)
         return {prefix + self.spec.weight_name: shape if self.spec.weight_offset else ScaleShape(shape)}
 
     def bind(self, prefix, weights):
@@ -31,6 +31,8 @@ class RMSNorm(Part):
             self.weight = (stored.to(device=self.device, dtype=torch.float32) + float(self.spec.weight_offset)).contiguous()
         else:
             self.weight = self.vector(stored)
+        if self.spec.one_weight:  # one number for all features: the kernels read a weight per feature
+            self.weight = self.weight.reshape(1).expand(self.spec.size).contiguous()
 
     def folded_for(self, rows: int):
         """(weight, eps) if, in a step of `rows` rows, whatever writes the residual before this norm

@@ -1,4 +1,4 @@
-"""Rotary position encoding (pairs (i, i + rot/2)).
+"""Rotary position encoding (pairs (i, i + rot/2), or neighbours; frequencies plain or stretched).
 
 inv_freq[i] = 1 / theta ** (2 i / rot), built exactly as the reference builds it
 (engine/model.py:132-135: int64 arange -> float, divided by the size, theta to
@@ -32,8 +32,13 @@ class NeoxRope(Part):
         rot = spec.rotary_dim
         if rot % 2:
             raise ValueError(f"rotary_dim {rot} must be even")
-        exponent = torch.arange(0, rot, 2, dtype=torch.int64).to(torch.float32)
-        self.inv_freq = (1.0 / (spec.theta ** (exponent / rot))).to(device)
+        self.magnitude = 1.0  # what cosines and sines are multiplied by
+        if spec.ramp is None:
+            exponent = torch.arange(0, rot, 2, dtype=torch.int64).to(torch.float32)
+            self.inv_freq = (1.0 / (spec.theta ** (exponent / rot))).to(device)
+        else:
+            freq, self.magnitude = ramped_frequencies(rot, spec.theta, spec.ramp)
+            self.inv_freq = freq.to(device)
 
     def rotary_table(self, ctx):
         """(rotated width, cosines and sines [T, width / 2, 2] of every token's angles): computed by
@@ -41,7 +46,7 @@ class NeoxRope(Part):
         rot = self.spec.rotary_dim
         if not rot:
             return 0, None
-        key = ("neox_rope", rot, self.spec.theta)
+        key = ("neox_rope", rot, self.spec.theta, self.spec.ramp)
         table = ctx.memo.get(key)
         if table is None:
             table = ctx.memo[key] = K.rope_table(ctx.positions, self.inv_freq)
@@ -50,7 +55,10 @@ class NeoxRope(Part):
     def encode(self, ctx, x: torch.Tensor, num_heads: int, head_dim: int) -> None:
         """Rotate the first `num_heads` heads of every row of `x` in place."""
         rot, table = self.rotary_table(ctx)
-        if rot:
+        if rot and self.magnitude != 1.0:
+            K.qk_norm_rotate_store(x, num_heads, 0, head_dim, head_dim, None, None, 0.0, rot, False, table,
+                                   self.magnitude, ctx.positions, None, None, 1, None, None)
+        elif rot:
             K.rotate_heads(x, num_heads, head_dim, rot, table, ctx.positions)
 
 

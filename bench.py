@@ -166,11 +166,33 @@ def zikezen_shape(shape: dict, layers: int) -> dict:
     return out
 
 
+def getodra_shape(shape: dict, layers: int) -> dict:
+    """A Getodra configuration with the layer sizes of the Qwen2.5 shape `shape`: the same width, feed-forward and
+    vocabulary; in turn lightning attention (as many heads of the same size, values as wide, decays from 0.6 to 0.9998) and
+    latent attention (as many heads: the head size unrotated and half of it rotated with stretched frequencies,
+    values of the head size, a latent of four head sizes, as in the Ritalorn shape); convolutions of four taps in front
+    of every sublayer; learned positions; in models of six layers or more the sixth uses the fourth's tensors."""
+    heads, hd = shape["num_attention_heads"], shape["head_dim"]
+    mlp = {"kind": "dense", "ff": shape["intermediate_size"]}
+    lightning = {"type": "lightning", "mlp": mlp, "mixer": {
+        "heads": heads, "dim": hd, "vdim": hd, "decay": [1.0 - 0.4 * 2.0 ** (-11.0 * h / max(1, heads - 1)) for h in range(heads)]}}
+    latent = {"type": "latent_attention", "mlp": mlp, "mixer": {
+        "heads": heads, "dim": hd, "rot_dim": hd // 2, "vdim": hd, "kv_rank": 4 * hd, "scale": (hd + hd // 2) ** -0.5,
+        "rot": {"base": float(shape["rope_theta"]), "dims": hd // 2,
+                "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    out = [dict(latent if i % 2 else lightning) for i in range(layers)]
+    if layers >= 6:
+        out[5]["weights_of"] = 3
+    return {"architecture": "Getodra", "vocab": shape["vocab_size"], "width": shape["hidden_size"],
+            "max_positions": int(shape.get("max_position_embeddings") or 32768), "norm": {"eps": shape["rms_norm_eps"]},
+            "canon": {"taps": 4}, "layers": out}
+
+
 def design_run(args, shape: dict) -> int:
-    """`--design danonex|ritalorn|dagavik|zikezen`: decode steps (batch 1, 8, 64 at the context asked for) and prefills of
+    """`--design danonex|ritalorn|dagavik|zikezen|getodra`: decode steps (batch 1, 8, 64 at the context asked for) and prefills of
     2,048 and 8,192 tokens of a model of that design with the shape's layer sizes, and beside each the same
     measurement of the Qwen2.5 shape (and, for ritalorn and dagavik, of the Danonex shape; for zikezen, of the Dagavik
-    shape) with the same number of layers (for zikezen: of layer runs).  One JSON line."""
+    shape; for getodra, of the Ritalorn and Zikezen shapes) with the same number of layers (for zikezen: of layer runs).  One JSON line."""
     import torch
 
     layers = args.layers or 8
@@ -179,7 +201,12 @@ def design_run(args, shape: dict) -> int:
                         f"prefill tok/s", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
               "dtype": "bf16" if args.dtype == "bfloat16" else "fp32", "context": args.ctx,
               "data": "synthetic: seeded uniform token ids, random weights N(0, 0.02)", "designs": {}}
-    if args.design == "zikezen":
+    if args.design == "getodra":
+        configs = {"getodra": getodra_shape(shape, layers)}
+        if not args.alone:
+            configs.update({"ritalorn": ritalorn_shape(shape, layers), "zikezen": zikezen_shape(shape, layers),
+                            "qwen2": dict(shape, num_hidden_layers=layers)})
+    elif args.design == "zikezen":
         configs = {"zikezen": zikezen_shape(shape, layers)}
         if not args.alone:
             configs.update({"dagavik": dagavik_shape(shape, layers), "qwen2": dict(shape, num_hidden_layers=layers)})
@@ -441,12 +468,12 @@ def main() -> int:
     parser.add_argument("--dtype", choices=("bfloat16", "float32"), default="bfloat16")
     parser.add_argument("--no-points", action="store_true", help="skip the batch 1 / 64 and prefill runs")
     parser.add_argument("--prefill-only", action="store_true", help="time the 2,048-token prefill alone (for profiles)")
-    parser.add_argument("--design", choices=("qwen2", "danonex", "ritalorn", "dagavik", "zikezen"), default="qwen2",
-                        help="danonex, ritalorn, dagavik, zikezen: a model of that design with the shape's layer sizes (8 layers "
+    parser.add_argument("--design", choices=("qwen2", "danonex", "ritalorn", "dagavik", "zikezen", "getodra"), default="qwen2",
+                        help="danonex, ritalorn, dagavik, zikezen, getodra: a model of that design with the shape's layer sizes (8 layers "
                              "unless --layers says otherwise) beside the Qwen2.5 shape (ritalorn, dagavik: and the Danonex shape; "
-                             "zikezen: and the Dagavik shape) with as many layers: decode at batch 1, 8, 64 and prefills of 2,048 "
-                             "and 8,192 tokens")
-    parser.add_argument("--alone", action="store_true", help="with --design ritalorn, dagavik or zikezen: that design only (for profiles)")
+                             "zikezen: and the Dagavik shape; getodra: and the Ritalorn and Zikezen shapes) with as many layers: "
+                             "decode at batch 1, 8, 64 and prefills of 2,048 and 8,192 tokens")
+    parser.add_argument("--alone", action="store_true", help="with --design ritalorn, dagavik, zikezen or getodra: that design only (for profiles)")
     args = parser.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU only: this engine has no multi-GPU path (run with --gpus 1)")
@@ -457,7 +484,7 @@ def main() -> int:
         print("bench.py needs a GPU", file=sys.stderr)
         return 1
     shape = QWEN25_1P5B if args.model == "1.5b" else OTHER_SHAPES[args.model]
-    if args.design in ("danonex", "ritalorn", "dagavik", "zikezen"):
+    if args.design in ("danonex", "ritalorn", "dagavik", "zikezen", "getodra"):
         try:
             return design_run(args, shape)
         except (Refused, Unresolved) as err:

@@ -99,6 +99,20 @@ int pae_latent_attn_bf16(void* out, int64_t out_stride, const void* q, int64_t q
                          int chunked, float* part_acc, float* part_ml, const float* sinks, const void* head_gate,
                          int64_t gate_stride, hipStream_t stream);
 int pae_latent_attn_split();
+// latent attention over long runs with the heads' keys and values formed: see latent_expand.hip
+int pae_latent_gather(void* rows, const void* latent, const int* pages, int num_pages, const int* block_tables,
+                      int max_blocks, int bs, int rank, int width, hipStream_t stream);
+int pae_latent_expand(void* keys, void* values, const void* up, int64_t up_stride, const void* latent, const int* pages,
+                      int num_pages, const int* block_tables, int max_blocks, int bs, int H, int D, int rd, int V, int rank,
+                      int KD, hipStream_t stream);
+int pae_latent_queries(void* out, const void* proj, int64_t row_stride, int num_tokens, const float* cos_sin,
+                       float magnitude, int H, int D, int rd, int rot, int interleaved, int KD, hipStream_t stream);
+// prefill attention with value heads of their own width and a gate per token and head: see attention_mfma.hip
+int pae_attn_prefill_wide_width(int width, int vd);
+int pae_attn_prefill_wide_bf16(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* k_cache,
+                               const void* v_cache, const int* tiles, int num_tiles, const int* positions,
+                               const int* block_tables, int max_blocks, int nh, int nkv, int hd, int vd, float scale,
+                               int window, const void* head_gate, int64_t head_gate_stride, hipStream_t stream);
 // rows [q | k | v]: RMS norm of q and of k over the whole projection, or head by head with one weight that the
 // heads share (`per_head`; weights null: none), rotation, cache write
 int pae_qk_norm_rotate_store(int dtype, void* qkv, int64_t row_stride, int num_tokens, int nh, int nkv, int hd, int vd,

@@ -274,16 +274,19 @@ __device__ __forceinline__ bf16x8 quad_to_mfma_order(bf16x8 x, int fetch_from) {
 // tiles[t] = (table row of the sequence, first flat token, number of tokens <= 64); blockIdx.z picks
 // the part of 16 CT tokens of the run that this workgroup takes.
 // BS: the page size if it is 16 (the value rows' offsets are then constants), or 0 for any other.
-template <int HD, int CT, int BS, bool CAPPED, bool BIASED>
+// VD: the width of a value head, if it is not HD.
+// `head_gate` (null: none): one number a token and head, the head's output is multiplied by its sigmoid.
+template <int HD, int CT, int BS, bool CAPPED, bool BIASED, int VD = HD>
 __global__ __launch_bounds__(256, 1) void attn_prefill_split_kernel(
     bf16_t* __restrict__ out, int64_t out_stride, const bf16_t* __restrict__ q, int64_t q_stride,
     const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache, const int* __restrict__ tiles,
     const int* __restrict__ positions, const int* __restrict__ block_tables, int max_blocks, int bs, int nh,
     int nkv, float scale_log2, int window, float cap_over_scale, float scale_over_cap, const float* __restrict__ sinks,
-    int chunked, const float* __restrict__ slopes, float inv_scale, const bf16_t* __restrict__ gate, int64_t gate_stride) {
+    int chunked, const float* __restrict__ slopes, float inv_scale, const bf16_t* __restrict__ gate, int64_t gate_stride,
+    const bf16_t* __restrict__ head_gate, int64_t head_gate_stride) {
   constexpr int UNIT = 32, TOK = 16 * CT;
   if (BS) bs = BS;
-  __shared__ float s_acc[3][HD / 16][4][PAE_WAVE];
+  __shared__ float s_acc[3][VD / 16][4][PAE_WAVE];
   __shared__ float s_ml[3][2][PAE_WAVE];
 
   // the wavefront's number as a scalar: what is computed from it (the keys it takes, their pages'
@@ -324,14 +327,14 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_split_kernel(
   const int last_start = BIASED ? first_visible(hi, window, chunked)
                                 : ((window > 0 && hi - window + 1 > 0) ? hi - window + 1 : 0);  // window start of the last token
 
-  f32x4 acc[CT][HD / 16];  // O^T: rows hd = 16 t + 4 g4 + i, column = lane % 16
+  f32x4 acc[CT][VD / 16];  // O^T: rows 16 t + 4 g4 + i, column = lane % 16
   float ref[CT], l[CT];    // the column's reference (log2 units) and this lane's share of its sum of weights
 #pragma unroll
   for (int ct = 0; ct < CT; ++ct) {
     ref[ct] = NEG_BIG;
     l[ct] = 0.f;
 #pragma unroll
-    for (int t = 0; t < HD / 16; ++t) acc[ct][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int t = 0; t < VD / 16; ++t) acc[ct][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
   }
 
   // Keys are loaded in the order (row = lane / 4, group = lane % 4), in which a quad of lanes reads
@@ -344,19 +347,18 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_split_kernel(
   // are exactly the scores the lane holds after the first product.
   const int lrow = lane / 4, lgrp = lane % 4;
   const int fetch_from = ((lane % 16) * 4 + lane / 16) * 4;
-  const int page_elems = bs * HD;
-  bf16x8 kf[2][HD / 32], vf[HD / 16];
-  auto page_base = [&](int key0, int p) -> int64_t {
+  bf16x8 kf[2][HD / 32], vf[VD / 16];
+  auto page_of = [&](int key0, int p) -> int64_t {  // in units of one head's page
     const int key = key0 + 16 * p;
     const int kc = key <= hi ? key : key0;  // a tile past the end repeats the first one (all of it is masked)
     // a page the window has passed was given back (its entry is -1): all its keys are masked, read page 0
-    return ((int64_t)max(table[kc / bs], 0) * nkv + kvh) * page_elems;
+    return (int64_t)max(table[kc / bs], 0) * nkv + kvh;
   };
   auto load_keys = [&](int key0) {
 #pragma unroll
     for (int p = 0; p < 2; ++p) {
       const int key = key0 + 16 * p, kc = key <= hi ? key : key0;
-      const bf16_t* kp = k_cache + page_base(key0, p) + (int64_t)(kc % bs) * HD;
+      const bf16_t* kp = k_cache + page_of(key0, p) * (bs * HD) + (int64_t)(kc % bs) * HD;
 #pragma unroll
       for (int j = 0; j < HD / 32; ++j) kf[p][j] = *reinterpret_cast<const bf16x8*>(kp + lrow * HD + 32 * j + 8 * lgrp);
     }
@@ -366,10 +368,10 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_split_kernel(
 #pragma unroll
     for (int p = 0; p < 2; ++p) {
       const int key = key0 + 16 * p, kc = key <= hi ? key : key0;
-      vp[p] = v_cache + page_base(key0, p) + kc % bs;
+      vp[p] = v_cache + page_of(key0, p) * (bs * VD) + kc % bs;
     }
 #pragma unroll
-    for (int t = 0; t < HD / 16; ++t)  // in the order of their use
+    for (int t = 0; t < VD / 16; ++t)  // in the order of their use
 #pragma unroll
       for (int p = 0; p < 2; ++p)
         reinterpret_cast<bf16x4*>(&vf[t])[p] = *reinterpret_cast<const bf16x4*>(vp[p] + (int64_t)(16 * t + col) * bs + 4 * g4);
@@ -455,7 +457,7 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_split_kernel(
 #pragma unroll
       for (int ct = 0; ct < CT; ++ct)
 #pragma unroll
-        for (int t = 0; t < HD / 16; ++t) asm volatile("" : "+a"(acc[ct][t]));  // moved from there only in here
+        for (int t = 0; t < VD / 16; ++t) asm volatile("" : "+a"(acc[ct][t]));  // moved from there only in here
 #pragma unroll
       for (int ct = 0; ct < CT; ++ct) {
         float m = fmaxf(mx[ct], NEG_BIG);
@@ -466,7 +468,7 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_split_kernel(
         ref[ct] = to;
         l[ct] *= alpha;
 #pragma unroll
-        for (int t = 0; t < HD / 16; ++t) acc[ct][t] *= alpha;
+        for (int t = 0; t < VD / 16; ++t) acc[ct][t] *= alpha;
       }
     }
     // the sums are in the accumulation registers on both ways here (or the compiler moves the whole
@@ -474,7 +476,7 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_split_kernel(
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct)
 #pragma unroll
-      for (int t = 0; t < HD / 16; ++t) asm volatile("" : "+a"(acc[ct][t]));
+      for (int t = 0; t < VD / 16; ++t) asm volatile("" : "+a"(acc[ct][t]));
     // Column tile by column tile: the weights of one (exponentials, sum, rounding: vector ALU), then
     // its second product (matrix pipe), so that the next tile's arithmetic can run under this
     // tile's products.
@@ -492,14 +494,14 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_split_kernel(
 #pragma unroll
       for (int i = 0; i < 4; ++i) pairs[i] = __builtin_convertvector((f32x2){w[2 * i], w[2 * i + 1]}, bf16x2);
 #pragma unroll
-      for (int t = 0; t < HD / 16; ++t) acc[ct][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[t], pb, acc[ct][t], 0, 0, 0);
+      for (int t = 0; t < VD / 16; ++t) acc[ct][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[t], pb, acc[ct][t], 0, 0, 0);
     }
     // Order asked of the compiler's scheduler for the above: the first tile's arithmetic, then one
     // matrix instruction and two vector instructions in turn (left alone it puts all exponentials
     // first and all products last, and each pipe idles while the other runs).
     __builtin_amdgcn_sched_group_barrier(0x002, 20, 0);
 #pragma unroll
-    for (int i = 0; i < CT * (HD / 16); ++i) {
+    for (int i = 0; i < CT * (VD / 16); ++i) {
       __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
       __builtin_amdgcn_sched_group_barrier(0x002, 2, 0);
     }
@@ -520,7 +522,7 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_split_kernel(
     if (wave != merger) {
       const int slot = wave < merger ? wave : wave - 1;
 #pragma unroll
-      for (int t = 0; t < HD / 16; ++t)
+      for (int t = 0; t < VD / 16; ++t)
 #pragma unroll
         for (int i = 0; i < 4; ++i) s_acc[slot][t][i][lane] = acc[ct][t][i];
       s_ml[slot][0][lane] = ref[ct];
@@ -544,15 +546,17 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_split_kernel(
       }
       const int c = ct * 16 + col;
       if (c < ntok) {
-        const float inv = 1.0f / sum;
-        bf16_t* o = out + (int64_t)(tok0 + c) * out_stride + (int64_t)head * HD;
-        const bf16_t* gt = (BIASED && gate) ? gate + (int64_t)(tok0 + c) * gate_stride + (int64_t)head * HD + 4 * g4 : nullptr;
-        s16x4 gates[HD / 16];  // four gate features per slice of 16, asked for together before the sums are formed
+        float inv = 1.0f / sum;
+        if (!BIASED && head_gate)
+          inv *= __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-__bfloat162float(head_gate[(int64_t)(tok0 + c) * head_gate_stride + head]) * LOG2E));
+        bf16_t* o = out + (int64_t)(tok0 + c) * out_stride + (int64_t)head * VD;
+        const bf16_t* gt = (BIASED && gate) ? gate + (int64_t)(tok0 + c) * gate_stride + (int64_t)head * VD + 4 * g4 : nullptr;
+        s16x4 gates[VD / 16];  // four gate features per slice of 16, asked for together before the sums are formed
         if (BIASED && gt)
 #pragma unroll
-          for (int t = 0; t < HD / 16; ++t) gates[t] = *reinterpret_cast<const s16x4*>(gt + 16 * t);
+          for (int t = 0; t < VD / 16; ++t) gates[t] = *reinterpret_cast<const s16x4*>(gt + 16 * t);
 #pragma unroll
-        for (int t = 0; t < HD / 16; ++t) {
+        for (int t = 0; t < VD / 16; ++t) {
           s16x4 w4;
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
@@ -710,7 +714,7 @@ static int attn_prefill_any(void* out, int64_t out_stride, const void* q, int64_
   attn_prefill_split_kernel<HD, CT, BS, CAPPED, BIASED><<<dim3(nh, num_tiles, 4 / CT), 256, 0, stream>>>(      \
       (bf16_t*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,    \
       tiles, positions, block_tables, max_blocks, bs, nh, nkv, scale_log2, window, cap_over_scale,             \
-      scale_over_cap, sinks, chunked, slopes, slopes ? 1.0f / scale : 0.f, (const bf16_t*)gate, gate_stride)
+      scale_over_cap, sinks, chunked, slopes, slopes ? 1.0f / scale : 0.f, (const bf16_t*)gate, gate_stride, nullptr, 0)
 #define LAUNCH_CT(HD, CT, BS)                  \
   if (biased) {                                \
     LAUNCH_CAPPED(HD, CT, BS, false, true);    \
@@ -765,4 +769,41 @@ extern "C" int pae_attn_prefill_bf16(void* out, int64_t out_stride, const void* 
                                      int nkv, int hd, float scale, int window, hipStream_t stream) {
   return pae_attn_prefill_capped_bf16(out, out_stride, q, q_stride, k_cache, v_cache, tiles, num_tiles, positions,
                                       block_tables, max_blocks, bs, nh, nkv, hd, scale, window, 0.f, nullptr, stream);
+}
+
+// Key widths `hd` (multiples of 32 up to 256) built for values `vd` wide: the smallest that holds `width` features, or 0.
+// Two column tiles (32 tokens) a workgroup.
+#define FOR_WIDE_SHAPE(CALL) CALL(64, 32) CALL(64, 64) CALL(96, 64) CALL(128, 64) CALL(128, 128) CALL(160, 128) CALL(192, 128) CALL(256, 128) CALL(256, 192)
+extern "C" int pae_attn_prefill_wide_width(int width, int vd) {
+#define WIDE_FITS(HD, VD) \
+  if (vd == VD && width <= HD) return HD;
+  FOR_WIDE_SHAPE(WIDE_FITS)
+#undef WIDE_FITS
+  return 0;
+}
+
+// `pae_attn_prefill_bf16` over pages of 16 with value heads of their own width and a gate per token and head.
+extern "C" int pae_attn_prefill_wide_bf16(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* k_cache,
+                                          const void* v_cache, const int* tiles, int num_tiles, const int* positions,
+                                          const int* block_tables, int max_blocks, int nh, int nkv, int hd, int vd, float scale,
+                                          int window, const void* head_gate, int64_t head_gate_stride, hipStream_t stream) {
+  if (int rc = check_common("attn_prefill_wide", nh, nkv, hd, 16, max_blocks, window)) return rc;
+  PAE_REQUIRE(pae_attn_prefill_wide_width(hd, vd) == hd, "attn_prefill_wide: keys of %d with values of %d are not built", hd, vd);
+  PAE_REQUIRE(out_stride >= (int64_t)nh * vd && q_stride >= (int64_t)nh * hd, "attn_prefill_wide: row strides too small");
+  PAE_REQUIRE(!head_gate || head_gate_stride >= nh, "attn_prefill_wide: gate row stride %lld too small", (long long)head_gate_stride);
+  PAE_REQUIRE(num_tiles <= 65535, "attn_prefill_wide: %d runs exceed the grid", num_tiles);
+  if (num_tiles <= 0) return 0;
+#define WIDE_LAUNCH(HD, CT, VD)                                                                                          \
+  attn_prefill_split_kernel<HD, CT, 16, false, false, VD><<<dim3(nh, num_tiles, 4 / CT), 256, 0, stream>>>(               \
+      (bf16_t*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, tiles,        \
+      positions, block_tables, max_blocks, 16, nh, nkv, scale * LOG2E, window, 0.f, 0.f, nullptr, 0, nullptr, 0.f, nullptr, 0, \
+      (const bf16_t*)head_gate, head_gate_stride)
+#define WIDE_CASE(HD, VD)                  \
+  if (hd == HD && vd == VD) {              \
+    WIDE_LAUNCH(HD, 2, VD);                \
+  }
+  FOR_WIDE_SHAPE(WIDE_CASE)
+#undef WIDE_CASE
+#undef WIDE_LAUNCH
+  return pae_check_launch("attn_prefill_wide");
 }

@@ -12,7 +12,8 @@
 //     all rd behind the latent;
 //   * rotates the last rd features of every query head likewise and writes them to
 //     q_full[t][head][kv_rank .. kv_rank + rd), where the attention kernel expects them behind the
-//     head's query folded into latent space (a product that the caller launches).
+//     head's query folded into latent space (a product that the caller launches); without q_full the queries
+//     are left alone.
 // The attention over the pages then scores q_full against the cached row as a whole,
 //   score = q_folded . c + q_rotated . k_rotated,
 // and takes its values from the first kv_rank features of the same row.
@@ -44,9 +45,9 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
     if (latent_t) latent_t[(block * rank + i) * bs + pos % bs] = c;
   }
   // rotated parts: "head" nh is the shared key part, heads 0 .. nh - 1 the queries'
-  const int half = rot / 2;
-  for (int idx = threadIdx.x; idx < (nh + 1) * half; idx += 256) {
-    const int h = idx / half, i = idx % half;
+  const int half = rot / 2, h0 = q_full ? 0 : nh;
+  for (int idx = threadIdx.x; idx < (nh + 1 - h0) * half; idx += 256) {
+    const int h = h0 + idx / half, i = idx % half;
     const int ia = interleaved ? 2 * i : i, ib = interleaved ? 2 * i + 1 : i + half;
     const float c = magnitude * cos_sin[((int64_t)t * half + i) * 2], s = magnitude * cos_sin[((int64_t)t * half + i) * 2 + 1];
     const T* src = h < nh ? row + (int64_t)h * (nope + rd) + nope : down + rank;
@@ -56,8 +57,8 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
     dst[ib] = from_f32<T>(b * c + a * s);
   }
   const int rest = rd - rot;  // features behind the rotated ones pass as they are
-  for (int idx = threadIdx.x; idx < (nh + 1) * rest; idx += 256) {
-    const int h = idx / rest, i = rot + idx % rest;
+  for (int idx = threadIdx.x; idx < (nh + 1 - h0) * rest; idx += 256) {
+    const int h = h0 + idx / rest, i = rot + idx % rest;
     const T* src = h < nh ? row + (int64_t)h * (nope + rd) + nope : down + rank;
     T* dst = h < nh ? q_full + (int64_t)t * qf_stride + (int64_t)h * (rank + rd) + rank : cached + rank;
     dst[i] = src[i];
@@ -75,8 +76,8 @@ extern "C" int pae_latent_prepare(int dtype, const void* proj, int64_t row_strid
   PAE_REQUIRE(rot == 0 || cos_sin, "latent_prepare: a rotation needs its table of cosines and sines");
   PAE_REQUIRE(row_stride >= (int64_t)nh * (nope + rd) + rank + rd, "latent_prepare: row stride %lld too small",
               (long long)row_stride);
-  PAE_REQUIRE(qf_stride >= (int64_t)nh * (rank + rd), "latent_prepare: query row stride %lld too small", (long long)qf_stride);
-  PAE_REQUIRE(bs > 0 && max_blocks > 0 && latent && block_tables && tok_seq && positions && norm_w && q_full,
+  PAE_REQUIRE(!q_full || qf_stride >= (int64_t)nh * (rank + rd), "latent_prepare: query row stride %lld too small", (long long)qf_stride);
+  PAE_REQUIRE(bs > 0 && max_blocks > 0 && latent && block_tables && tok_seq && positions && norm_w,
               "latent_prepare: missing operands");
   if (num_tokens <= 0) return 0;
   if (dtype == PAE_F32)

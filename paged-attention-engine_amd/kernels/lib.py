@@ -84,6 +84,11 @@ def _declare(lib) -> None:
         "pae_latent_attn_columns": [I, I],
         "pae_latent_attn_bf16": [P, L, P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, I, I, P, P, P, P, L, P],
         "pae_latent_attn_split": [],
+        "pae_latent_gather": [P, P, P, I, P, I, I, I, I, P],
+        "pae_latent_expand": [P, P, P, L, P, P, I, P, I, I, I, I, I, I, I, I, P],
+        "pae_latent_queries": [P, P, L, I, P, F, I, I, I, I, I, I, P],
+        "pae_attn_prefill_wide_width": [I, I],
+        "pae_attn_prefill_wide_bf16": [P, L, P, L, P, P, P, I, P, P, I, I, I, I, I, F, I, P, L, P],
         "pae_gated_act": [I, P, P, I, I, I, I, P],
         "pae_gemm_plain_batched": [I, I, P, L, L, P, L, L, P, L, P, I, I, I, I, I, P],
         "pae_rows_from_residual": [I, P, P, L, P],
@@ -1164,7 +1169,7 @@ def conv_norm_store(proj: torch.Tensor, q_out: torch.Tensor, tok_seq: torch.Tens
         _ptr(v_cache) if nkv else None, _stream()))
 
 
-def latent_prepare(proj: torch.Tensor, q_full: torch.Tensor, nh: int, nope: int, rd: int, rot: int, interleaved: bool,
+def latent_prepare(proj: torch.Tensor, q_full: Optional[torch.Tensor], nh: int, nope: int, rd: int, rot: int, interleaved: bool,
                    rank: int, norm_w: torch.Tensor, eps: float, cos_sin: Optional[torch.Tensor], positions: torch.Tensor,
                    tok_seq: torch.Tensor, block_tables: torch.Tensor, latent: torch.Tensor,
                    latent_t: Optional[torch.Tensor] = None, magnitude: float = 1.0) -> None:
@@ -1172,7 +1177,7 @@ def latent_prepare(proj: torch.Tensor, q_full: torch.Tensor, nh: int, nope: int,
     features of the down projection are RMS-normed with `norm_w` and, with the last rd (their first
     `rot` rotated by `cos_sin` times `magnitude`), written to the token's row of `latent` [block][bs][rank + rd]; the
     query heads' last rd features are rotated likewise into q_full[t, h, rank:] (`q_full`
-    [T, nh * (rank + rd)], whose first `rank` features per head the caller fills).  With `latent_t`
+    [T, nh * (rank + rd)], whose first `rank` features per head the caller fills; None: the queries are left alone).  With `latent_t`
     [block][rank][bs] the normed latents are also written transposed within the page."""
     _not_while_recording("latent_prepare")
     _gpu(proj, q_full, norm_w, cos_sin, positions, tok_seq, block_tables, latent, latent_t)
@@ -1181,7 +1186,8 @@ def latent_prepare(proj: torch.Tensor, q_full: torch.Tensor, nh: int, nope: int,
         assert latent_t.dtype == latent.dtype
     T = proj.shape[0]
     assert proj.dim() == 2 and proj.stride(1) == 1 and proj.shape[1] >= nh * (nope + rd) + rank + rd
-    assert q_full.shape == (T, nh * (rank + rd)) and q_full.stride(1) == 1 and q_full.dtype == proj.dtype
+    if q_full is not None:
+        assert q_full.shape == (T, nh * (rank + rd)) and q_full.stride(1) == 1 and q_full.dtype == proj.dtype
     assert latent.dim() == 3 and latent.shape[2] == rank + rd and latent.is_contiguous() and latent.dtype == proj.dtype
     assert positions.dtype == torch.int32 and positions.numel() == T
     assert tok_seq.dtype == torch.int32 and tok_seq.numel() == T
@@ -1190,8 +1196,8 @@ def latent_prepare(proj: torch.Tensor, q_full: torch.Tensor, nh: int, nope: int,
     _check_cos_sin(cos_sin, rot, T)
     wp, wf = _param(norm_w)
     _check(library().pae_latent_prepare(
-        code_of(proj.dtype), proj.data_ptr(), proj.stride(0), q_full.data_ptr(), q_full.stride(0), T, nh, nope, rd, rot,
-        1 if interleaved else 0, rank, wp, wf, float(eps), _ptr(cos_sin) if rot else None, float(magnitude),
+        code_of(proj.dtype), proj.data_ptr(), proj.stride(0), _ptr(q_full), q_full.stride(0) if q_full is not None else 0, T,
+        nh, nope, rd, rot, 1 if interleaved else 0, rank, wp, wf, float(eps), _ptr(cos_sin) if rot else None, float(magnitude),
         positions.data_ptr(), tok_seq.data_ptr(), block_tables.data_ptr(), block_tables.shape[1], latent.shape[1], latent.data_ptr(),
         _ptr(latent_t), _stream()))
 
@@ -1242,6 +1248,58 @@ def latent_attn(out: torch.Tensor, q_full: torch.Tensor, latent: torch.Tensor, l
         out.data_ptr(), out.stride(0), q_full.data_ptr(), q_full.stride(0), latent.data_ptr(), latent_t.data_ptr(),
         tiles.data_ptr(), tiles.shape[0], column_tiles, positions.data_ptr(), block_tables.data_ptr(), block_tables.shape[1],
         bs, nh, kd, rank, float(scale), int(window), 1 if chunked else 0, _ptr(part_acc), _ptr(part_ml), _ptr(sinks),
+        _ptr(head_gate), head_gate.stride(0) if head_gate is not None else 0, _stream()))
+
+
+def latent_key_width(dtype: torch.dtype, row_width: int, rank: int, head_width: int, value_dim: int) -> int:
+    """Width of the key rows in which `latent_expanded` keeps heads of `head_width` features (0: it does not take them)."""
+    if dtype != torch.bfloat16 or row_width % 8 or rank % 8 or head_width % 2 or value_dim % 2:
+        return 0
+    return library().pae_attn_prefill_wide_width(int(head_width), int(value_dim))
+
+
+def latent_expanded(out: torch.Tensor, proj: torch.Tensor, latent: torch.Tensor, up_weight: torch.Tensor, pages: torch.Tensor,
+                    page_table: torch.Tensor, tiles: torch.Tensor, positions: torch.Tensor, block_tables: torch.Tensor,
+                    cos_sin: Optional[torch.Tensor], magnitude: float, nh: int, nope: int, rd: int, rot: int, interleaved: bool,
+                    value_dim: int, rank: int, scale: float, head_gate: Optional[torch.Tensor] = None) -> None:
+    """Latent attention for runs of many tokens, the heads' keys and values formed first: out[t, h * value_dim:] of
+    the runs' tokens receives the heads (gated by sigmoid of `head_gate` [T, >= nh] if given); other rows are left alone.
+    `proj` and `latent` as for `latent_prepare`, which has written the runs' rows; `up_weight` [nh (nope + value_dim),
+    rank] = [W_uk; W_uv].  `pages` int32 [n, 4] = (table row of the sequence, position of the first key, keys, 0) cuts
+    every run's keys, from the sequence's first on, into pages of 16; `page_table` int32 [runs, width] names each run's
+    pages in that list, in order; `tiles` int32 [m, 3] = (row of `page_table`, first flat token, tokens <= PREFILL_TILE)."""
+    _not_while_recording("latent_expanded")
+    _gpu(out, proj, latent, up_weight, pages, page_table, tiles, positions, block_tables, cos_sin, head_gate)
+    T, n, bs = proj.shape[0], pages.shape[0], latent.shape[1]
+    width = latent_key_width(proj.dtype, latent.shape[2], rank, nope + rd, value_dim)
+    assert width > 0 and latent.shape[2] == rank + rd and latent.is_contiguous() and latent.dtype == proj.dtype == out.dtype
+    assert proj.dim() == 2 and proj.stride(1) == 1 and proj.shape[1] >= nh * (nope + rd)
+    assert out.shape == (T, nh * value_dim) and out.stride(1) == 1
+    assert up_weight.shape == (nh * (nope + value_dim), rank) and up_weight.is_contiguous() and up_weight.dtype == proj.dtype
+    for lists, columns in ((pages, 4), (page_table, None), (tiles, 3)):
+        assert lists.dtype == torch.int32 and lists.dim() == 2 and lists.is_contiguous()
+        assert columns is None or lists.shape[1] == columns
+    assert pages.data_ptr() % 16 == 0 and n > 0
+    assert positions.dtype == torch.int32 and positions.numel() == T
+    assert block_tables.dtype == torch.int32 and block_tables.dim() == 2 and block_tables.is_contiguous()
+    _check_cos_sin(cos_sin, rot, T)
+    if head_gate is not None:
+        _check_head_gate(head_gate, proj, nh)
+    lib, new = library(), lambda *shape: torch.empty(shape, dtype=proj.dtype, device=proj.device)
+    rows = new(n * 16, rank)
+    _check(lib.pae_latent_gather(rows.data_ptr(), latent.data_ptr(), pages.data_ptr(), n, block_tables.data_ptr(),
+                                 block_tables.shape[1], bs, rank, rank + rd, _stream()))
+    up = torch.mm(rows, up_weight.t())
+    keys, values = new(n, nh, 16, width), new(n, nh, value_dim, 16)
+    _check(lib.pae_latent_expand(keys.data_ptr(), values.data_ptr(), up.data_ptr(), up.stride(0), latent.data_ptr(),
+                                 pages.data_ptr(), n, block_tables.data_ptr(), block_tables.shape[1], bs, nh, nope, rd,
+                                 value_dim, rank, width, _stream()))
+    q = new(T, nh * width)
+    _check(lib.pae_latent_queries(q.data_ptr(), proj.data_ptr(), proj.stride(0), T, _ptr(cos_sin) if rot else None,
+                                  float(magnitude), nh, nope, rd, rot, 1 if interleaved else 0, width, _stream()))
+    _check(lib.pae_attn_prefill_wide_bf16(
+        out.data_ptr(), out.stride(0), q.data_ptr(), q.stride(0), keys.data_ptr(), values.data_ptr(), tiles.data_ptr(),
+        tiles.shape[0], positions.data_ptr(), page_table.data_ptr(), page_table.shape[1], nh, nh, width, value_dim, float(scale), 0,
         _ptr(head_gate), head_gate.stride(0) if head_gate is not None else 0, _stream()))
 
 

@@ -23,6 +23,11 @@ space once per token ([W_uk_j^T q_nope | q_rot], kv_rank + rope_dim wide), the a
 it against the cached row as it is and sums the rows' first kv_rank features as values, and the
 head's output is W_uv_j times that sum.  The query projection and the down projection are one
 product (a gate's rows ride in it); the two per-head products are one launch each.
+
+That costs kv_rank + rope_dim multiply-adds a score and kv_rank a value, the least where few queries meet many keys.
+Runs of many tokens (`EXPAND_ROWS`, bfloat16, every earlier key visible) have their keys and values formed instead, in one
+product over the run's keys, and attend with heads of nope_dim + rope_dim and value_dim (`kernels.lib.latent_expanded`);
+the cache stays as it is.
 """
 
 from __future__ import annotations
@@ -44,11 +49,17 @@ def latent_pages(kv_rank: int, rope_dim: int, window=None, transposed: bool = Fa
     return PagedSpec(tensors, window)
 
 
-def latent_tiles(shape: StepShape, single: int, runs: int):
+EXPAND_ROWS = 128  # runs of at least this many tokens attend with the heads' keys and values formed
+
+
+def latent_tiles(shape: StepShape, single: int, runs: int, expand: int = 0):
     """Work lists of the matrix-core kernel: (table row, first flat token, tokens, 0) for every sequence that
-    brings one token (`single`), and for the others in pieces of up to `runs` tokens, those with the most keys first."""
+    brings one token (`single`), and for the others in pieces of up to `runs` tokens, those with the most keys first.
+    `expand` > 0: sequences that bring at least that many tokens are in the lists of `expanded_runs` instead."""
     one, many = [], []
     for row, (start, n, past) in enumerate(zip(shape.q_starts, shape.q_lens, shape.past_lens)):
+        if expand and n >= expand:
+            continue
         if n == 1:
             one += [row, start, 1, 0]
         else:
@@ -56,6 +67,25 @@ def latent_tiles(shape: StepShape, single: int, runs: int):
                 many.append((past + first, (row, start + first, min(runs, n - first), 0)))
     many.sort(key=lambda piece: -piece[0])
     return {"single": (one, 4), "runs": ([x for _, piece in many for x in piece], 4)}
+
+
+def expanded_runs(shape: StepShape, expand: int):
+    """Work lists of `kernels.lib.latent_expanded` for the sequences that bring at least `expand` tokens."""
+    pages, tables, pieces = [], [], []
+    for row, (start, n, past) in enumerate(zip(shape.q_starts, shape.q_lens, shape.past_lens)):
+        if n < expand:
+            continue
+        first, keys = len(pages) // 4, past + n
+        for at in range(0, keys, 16):
+            pages += [row, at, min(16, keys - at), 0]
+        for at in range(0, n, K.PREFILL_TILE):
+            count = min(K.PREFILL_TILE, n - at)
+            pieces.append((past + at + count, (len(tables), start + at, count)))
+        tables.append(list(range(first, len(pages) // 4)))
+    pieces.sort(key=lambda piece: -piece[0])
+    width = max((len(t) for t in tables), default=1)
+    return {"pages": (pages, 4), "page_table": ([x for t in tables for x in t + [-1] * (width - len(t))], width),
+            "tiles": ([x for _, piece in pieces for x in piece], 3)}
 
 
 @register_mixer("latent_attention")
@@ -107,11 +137,20 @@ class LatentAttention(Part):
         if not (self.matrix_cores and block_size % 16 == 0):
             return None
         H = self.spec.num_heads
-        return ("latent attention tiles", K.latent_attn_tokens(H, 1), K.latent_attn_tokens(H, 2))
+        return ("latent attention tiles", K.latent_attn_tokens(H, 1), K.latent_attn_tokens(H, 2), self.expand_rows)
 
     def step_lists(self, shape: StepShape):
         H = self.spec.num_heads
-        return latent_tiles(shape, K.latent_attn_tokens(H, 1), K.latent_attn_tokens(H, 2))
+        lists = latent_tiles(shape, K.latent_attn_tokens(H, 1), K.latent_attn_tokens(H, 2), self.expand_rows)
+        return {**lists, **expanded_runs(shape, self.expand_rows)} if self.expand_rows else lists
+
+    @property
+    def expand_rows(self) -> int:
+        """Runs of at least this many tokens attend with the heads' keys and values formed (0: none do)."""
+        s = self.spec
+        takes = (s.own_kv and not s.window and not s.sinks and self.matrix_cores
+                 and K.latent_key_width(self.dtype, self.row_width, s.kv_rank, s.nope_dim + s.rope_dim, s.value_dim) > 0)
+        return EXPAND_ROWS if takes else 0
 
     def tensors(self, prefix):
         s = self.spec
@@ -143,14 +182,15 @@ class LatentAttention(Part):
         # sinks enter the softmax, which is float32
         self.sinks = (weights[prefix + s.sink_name].to(device=self.device, dtype=torch.float32).contiguous()
                       if s.sinks else None)
-        up_k = weights[prefix + s.up_k_name + sfx].view(s.num_heads, s.nope_dim, s.kv_rank)
+        # all heads' keys and values as one product of the latents, for runs of many tokens
+        self.up = self.matrix(torch.cat([weights[prefix + s.up_k_name + sfx], weights[prefix + s.up_v_name + sfx]], dim=0))
+        up_k, up_v = self.up.split([s.num_heads * s.nope_dim, s.num_heads * s.value_dim])
+        self.up_k = up_k.view(s.num_heads, s.nope_dim, s.kv_rank)
+        self.up_v = up_v.view(s.num_heads, s.value_dim, s.kv_rank)
         # the fold q_nope -> W_uk^T q_nope is a product with W_uk^T as its [out, in] matrix, head by head
-        self.up_k_t = self.matrix(up_k.transpose(1, 2))
-        self.up_v = self.matrix(weights[prefix + s.up_v_name + sfx].view(s.num_heads, s.value_dim, s.kv_rank))
-        # both the other way round as well, for steps of many rows (see kernels.lib.heads_product)
-        self.up_k = self.up_v_t = None
-        if self.dtype == torch.bfloat16:
-            self.up_k, self.up_v_t = self.matrix(up_k), self.matrix(self.up_v.transpose(1, 2))
+        self.up_k_t = self.up_k.transpose(1, 2).contiguous()
+        # and the values' the other way round, for steps of many rows (see kernels.lib.heads_product)
+        self.up_v_t = self.up_v.transpose(1, 2).contiguous() if self.dtype == torch.bfloat16 else None
         self.out = Linear(self.matrix(weights[prefix + s.o_name + sfx]))
 
     def forward(self, ctx, x):
@@ -168,23 +208,32 @@ class LatentAttention(Part):
             first = H * (D + R) + (C + R if s.own_kv else 0)
             gate = proj[:, first:first + H]
         rot, cos_sin = self.position.rotary_table(ctx)
-        q_full = torch.empty((T, H * (C + R)), dtype=proj.dtype, device=proj.device)
-        if s.own_kv:
-            K.latent_prepare(proj, q_full, H, D, R, rot, bool(getattr(self.position, "interleaved", False)), C,
-                             self.down_norm, s.norm_eps, cos_sin, ctx.positions, ctx.tok_seq, table, latent, latent_t,
-                             magnitude=float(getattr(self.position, "magnitude", 1.0)))
-        K.heads_product(q_full.view(T, H, C + R)[:, :, :C], proj[:, :H * (D + R)].view(T, H, D + R)[:, :, :D], self.up_k_t, self.up_k)
-        summed = torch.empty((T, H * C), dtype=proj.dtype, device=proj.device)
+        interleaved = bool(getattr(self.position, "interleaved", False))
+        magnitude = float(getattr(self.position, "magnitude", 1.0))
         key = self.step_lists_key(ctx.cache.block_size)
-        if key is not None and latent_t is not None:
-            tiles = ctx.memo[key]
-            for name, column_tiles in (("single", 1), ("runs", 2)):
-                if tiles[name].numel():
-                    K.latent_attn(summed, q_full, latent, latent_t, tiles[name], column_tiles, ctx.positions, table, H, C,
-                                  s.scale, s.window or 0, s.mask == "chunk", self.sinks, head_gate=gate)
-        else:
-            K.paged_attention_masked(summed, q_full, latent, None, ctx.positions, ctx.tok_seq, table, H, 1, C + R, C, s.scale,
-                                     s.window or 0, s.mask == "chunk", sinks=self.sinks, head_gate=gate)
+        tiles = ctx.memo[key] if key is not None and latent_t is not None else None
+        formed = tiles is not None and "pages" in tiles and tiles["pages"].numel() > 0
+        # do some rows meet the cached rows as they are?  (all but those of long runs)
+        folded = tiles is None or tiles["single"].numel() > 0 or tiles["runs"].numel() > 0
+        q_full = torch.empty((T, H * (C + R)), dtype=proj.dtype, device=proj.device) if folded else None
+        if s.own_kv:
+            K.latent_prepare(proj, q_full, H, D, R, rot, interleaved, C, self.down_norm, s.norm_eps, cos_sin, ctx.positions,
+                             ctx.tok_seq, table, latent, latent_t, magnitude=magnitude)
         heads = torch.empty((T, H * V), dtype=proj.dtype, device=proj.device)
-        K.heads_product(heads.view(T, H, V), summed.view(T, H, C), self.up_v, self.up_v_t)
+        if folded:
+            K.heads_product(q_full.view(T, H, C + R)[:, :, :C], proj[:, :H * (D + R)].view(T, H, D + R)[:, :, :D], self.up_k_t,
+                            self.up_k)
+            summed = torch.empty((T, H * C), dtype=proj.dtype, device=proj.device)
+            if tiles is not None:
+                for name, column_tiles in (("single", 1), ("runs", 2)):
+                    if tiles[name].numel():
+                        K.latent_attn(summed, q_full, latent, latent_t, tiles[name], column_tiles, ctx.positions, table, H, C,
+                                      s.scale, s.window or 0, s.mask == "chunk", self.sinks, head_gate=gate)
+            else:
+                K.paged_attention_masked(summed, q_full, latent, None, ctx.positions, ctx.tok_seq, table, H, 1, C + R, C,
+                                         s.scale, s.window or 0, s.mask == "chunk", sinks=self.sinks, head_gate=gate)
+            K.heads_product(heads.view(T, H, V), summed.view(T, H, C), self.up_v, self.up_v_t)
+        if formed:  # over whatever the products above made of these rows
+            K.latent_expanded(heads, proj, latent, self.up, tiles["pages"], tiles["page_table"], tiles["tiles"], ctx.positions,
+                              table, cos_sin, magnitude, H, D, R, rot, interleaved, V, C, s.scale, gate)
         return self.out.branch(heads, ctx.sink)

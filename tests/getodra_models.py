@@ -5,7 +5,7 @@ first, several of a kind in a row, layers that borrow an earlier layer's tensors
 each kind), layers without a feed-forward, convolutions of one to six taps, one head and several (more than a column
 tile of the matrix cores holds), key widths that take the recurrence in chunks of either length, value widths above and
 below the key width, decays close to one, one, one half and near zero, latents the matrix-core kernel takes and latents
-it does not, stretched frequencies (where some pairs keep theirs, some are blended and some divided) and plain ones,
+it does not, heads whose keys and values long runs form and heads whose they do not, stretched frequencies (where some pairs keep theirs, some are blended and some divided) and plain ones,
 widths the few-row product kernels take and widths they do not.  Weights are drawn so that no mechanism hides: filters
 a third of a unit wide, the latent norms and the lightning norms a fifth about one, the norms' single numbers spread
 about one, gates wide enough to open and shut, queries and keys wide enough that attention is peaked.
@@ -51,7 +51,7 @@ Q = {"architecture": "Getodra", "vocab": 211, "width": 100, "max_positions": 200
 # latents the matrix-core kernel takes, with more heads than one column tile holds and with fewer; two taps
 R = {"architecture": "Getodra", "vocab": 400, "width": 128, "max_positions": 512, "norm": {"eps": 1e-5}, "canon": {"taps": 2},
      "layers": [layer(latent(18, 16, 32, 16, 64, 0.2, base=3000.0, scaling=(4.0, 128, 16.0, 2.0)), 256),
-                layer(lightning(4, 32, 32, (0.5, 0.9, 0.99, 0.9999)), 128), layer(latent(6, 32, 32, 48, 128, 0.2, base=100.0), 96),
+                layer(lightning(4, 32, 32, (0.5, 0.9, 0.99, 0.9999)), 128), layer(latent(6, 32, 32, 32, 128, 0.2, base=100.0), 96),
                 layer(lightning(2, 128, 64, (0.7, 0.97)), 64)]}
 # nothing is a multiple of four; more taps than the register path holds
 S = {"architecture": "Getodra", "vocab": 97, "width": 90, "max_positions": 160, "norm": {"eps": 1e-5}, "canon": {"taps": 6},

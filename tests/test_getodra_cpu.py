@@ -152,6 +152,28 @@ def test_work_lists_of_the_convolutions_and_the_recurrence():
     assert lists["runs"] == ([0, 3, 40, 0, 3, 10, 5, 0], 4)
 
 
+def test_work_lists_of_latent_attention():
+    """Single tokens and short runs meet the cached rows as they are; sequences that bring many tokens have all their keys,
+    from the sequence's first on, cut into pages of 16 whose rows the heads' keys and values are formed in."""
+    from paged_attention_engine_amd.parts import StepShape
+    from paged_attention_engine_amd.parts.latent import expanded_runs, latent_tiles
+
+    shape = StepShape((7, 8, 9, 10), (0, 1, 131, 134), (1, 130, 3, 200), (40, 10, 0, 0), 16)
+    lists = latent_tiles(shape, 1, 2, 128)
+    assert lists["single"] == ([0, 0, 1, 0], 4)
+    assert lists["runs"] == ([2, 133, 1, 0, 2, 131, 2, 0], 4)
+    formed = expanded_runs(shape, 128)
+    pages, _ = formed["pages"]
+    assert pages[:8] == [1, 0, 16, 0, 1, 16, 16, 0] and pages[8 * 4:9 * 4] == [1, 128, 12, 0] and pages[9 * 4:10 * 4] == [3, 0, 16, 0]
+    assert len(pages) // 4 == 9 + 13
+    table, width = formed["page_table"]
+    assert width == 13 and table == list(range(9)) + [-1] * 4 + list(range(9, 22))
+    # pieces of 64 tokens, those with the most keys first, by their row in the table of pages
+    assert formed["tiles"] == ([1, 326, 8, 1, 262, 64, 0, 129, 2, 0, 65, 64, 1, 198, 64, 0, 1, 64, 1, 134, 64], 3)
+    assert latent_tiles(shape, 1, 2)["runs"][0][:4] == [3, 332, 2, 0]  # without the other kind every run is here
+    assert expanded_runs(StepShape((7,), (0,), (5,), (9,), 16), 128) == {"pages": ([], 4), "page_table": ([], 1), "tiles": ([], 3)}
+
+
 def test_the_bench_shape_is_a_config_the_reader_takes():
     """`bench.py --design getodra` builds its model from a config of its own making: as many layers as asked for."""
     import bench

@@ -231,11 +231,11 @@ def test_a_value_written_once_is_read_across_a_chunks_edge_and_far_back(D, chunk
 
 
 def latent_ways(lib, proj, w, H, D, R, V, C, bs, scale, base, scaling, dtype, new_from, gate):
-    """Heads [n, H * V] of the rows from `new_from` on, by the kernel for any shape and, where it takes the shape, by the
-    matrix-core kernels (single tokens and runs)."""
+    """Heads [n, H * V] of the rows from `new_from` on, by the kernel for any shape and, where they take the shape, by the
+    matrix-core kernels (single tokens and runs) and with the heads' keys and values formed."""
     from paged_attention_engine_amd.config.model_config import FrequencyRamp, PositionSpec
     from paged_attention_engine_amd.parts.base import POSITION_ENCODINGS
-    from paged_attention_engine_amd.parts.latent import latent_tiles
+    from paged_attention_engine_amd.parts.latent import expanded_runs, latent_tiles
 
     T = proj.shape[0]
     ramp = None if scaling is None else FrequencyRamp(**scaling)
@@ -275,6 +275,13 @@ def latent_ways(lib, proj, w, H, D, R, V, C, bs, scale, base, scaling, dtype, ne
                 lib.latent_attn(fast, q_full[new_from:], latent, latent_t, on_device(lists[name][0]), column_tiles, positions[new_from:],
                                 tables, H, C, scale, head_gate=gate[new_from:])
         finish("matrix cores", fast)
+    if cores and bs % 16 == 0 and lib.latent_key_width(dtype, C + R, C, D + R, V):
+        lists = expanded_runs(step_shape((n,), (new_from,), bs), 1)
+        heads = torch.zeros(n, H * V, dtype=dtype, device=DEV)
+        lib.latent_expanded(heads, proj[new_from:], latent, torch.cat([up_k.view(H * D, C), up_v.view(H * V, C)]),
+                            *(on_device(*lists[name]) for name in ("pages", "page_table", "tiles")), positions[new_from:], tables,
+                            cos_sin[new_from:].contiguous(), rope.magnitude, H, D, R, R, False, V, C, scale, gate[new_from:])
+        ways["keys and values formed"] = heads
     return ways
 
 
@@ -285,7 +292,9 @@ YARN = dict(factor=8.0, original=64.0, fast=8.0, slow=1.0)
 @pytest.mark.parametrize("H,D,R,V,C,bs,T,scaling", [(3, 16, 8, 24, 40, 16, 150, YARN), (2, 24, 16, 8, 16, 8, 70, None),
                                                     (4, 32, 32, 32, 64, 16, 330, YARN), (18, 16, 32, 16, 64, 32, 90, YARN),
                                                     (1, 40, 12, 72, 72, 16, 80, dict(factor=2.0, original=32.0, fast=4.0, slow=0.5)),
-                                                    (12, 16, 64, 16, 512, 16, 300, YARN)])
+                                                    (12, 16, 64, 16, 512, 16, 300, YARN), (5, 40, 32, 64, 96, 16, 210, YARN),
+                                                    (2, 128, 64, 128, 512, 16, 170, YARN), (3, 100, 32, 128, 64, 32, 140, None),
+                                                    (2, 192, 64, 192, 128, 16, 70, YARN), (1, 96, 32, 64, 160, 48, 100, None)])
 @pytest.mark.parametrize("new", ["prompt", "portion", "single"])
 def test_latent_attention_with_half_rotations_and_a_gate_per_head(dtype, H, D, R, V, C, bs, T, scaling, new):
     """Projected rows to gated heads against the plain mixer's keys and values formed head by head: pairs (i, i + R / 2), with
@@ -319,7 +328,7 @@ def test_latent_attention_with_half_rotations_and_a_gate_per_head(dtype, H, D, R
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("H,C,R,T", [(4, 64, 32, 300), (18, 64, 32, 40), (3, 40, 8, 90)])
+@pytest.mark.parametrize("H,C,R,T", [(4, 64, 32, 300), (18, 64, 32, 40), (3, 40, 8, 90), (2, 128, 32, 150)])
 def test_a_gate_that_shuts_every_head_but_one(dtype, H, C, R, T):
     """Gates of -60 leave nothing of a head, a gate of +60 leaves it whole, and 0 halves it: on prompts, on single tokens
     whose keys are split and merged (more than 256 of them), and by the kernel for any shape."""

@@ -125,11 +125,73 @@ __global__ __launch_bounds__(256) void heads_product_few_kernel(bf16_t* __restri
   }
 }
 
+// The same for inner sizes and strides in multiples of eight: eight numbers a load, L lanes an output feature (as many as
+// a row of eights needs, up to the wavefront), 64 / L features a wavefront.
+__device__ __forceinline__ void eight_of(const uint4& raw, float (&v)[8]) {  // a bfloat16 is the upper half of a float
+  const unsigned w[4] = {raw.x, raw.y, raw.z, raw.w};
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    v[2 * i] = __uint_as_float(w[i] << 16);
+    v[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
+  }
+}
+
+template <int L>
+__global__ __launch_bounds__(256) void heads_product_few_vec_kernel(bf16_t* __restrict__ out, int64_t ldc, int64_t head_c,
+                                                                    const bf16_t* __restrict__ a, int64_t lda, int64_t head_a,
+                                                                    const bf16_t* __restrict__ w, int M, int N, int K) {
+  const int lane = threadIdx.x % PAE_WAVE, wave = threadIdx.x / PAE_WAVE, sub = lane % L;
+  const int n = (blockIdx.x * 4 + wave) * (PAE_WAVE / L) + lane / L, h = blockIdx.y;
+  const bool live = n < N;  // dead groups run along: the sums below stay within a group of L lanes
+  const bf16_t* wr = w + ((int64_t)h * N + (live ? n : 0)) * K;
+  const bf16_t* ar = a + h * head_a;
+  for (int m0 = 0; m0 < M; m0 += HEADS_FEW_ROWS) {
+    float sum[HEADS_FEW_ROWS];
+#pragma unroll
+    for (int r = 0; r < HEADS_FEW_ROWS; ++r) sum[r] = 0.f;
+    for (int k = sub * 8; k < K; k += L * 8) {
+      const uint4 wraw = *reinterpret_cast<const uint4*>(wr + k);
+      uint4 araw[HEADS_FEW_ROWS];
+#pragma unroll
+      for (int r = 0; r < HEADS_FEW_ROWS; ++r)
+        if (m0 + r < M) araw[r] = *reinterpret_cast<const uint4*>(ar + (int64_t)(m0 + r) * lda + k);
+      float wv[8];
+      eight_of(wraw, wv);
+#pragma unroll
+      for (int r = 0; r < HEADS_FEW_ROWS; ++r)
+        if (m0 + r < M) {
+          float av[8];
+          eight_of(araw[r], av);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) sum[r] = fmaf(av[i], wv[i], sum[r]);
+        }
+    }
+#pragma unroll
+    for (int r = 0; r < HEADS_FEW_ROWS; ++r) {
+      if (m0 + r >= M) break;
+#pragma unroll
+      for (int off = L / 2; off > 0; off >>= 1) sum[r] += __shfl_xor(sum[r], off, L);
+      if (sub == 0 && live) out[(int64_t)(m0 + r) * ldc + h * head_c + n] = __float2bfloat16(sum[r]);
+    }
+  }
+}
+
 extern "C" int pae_heads_product_few(void* out, int64_t ldc, int64_t head_c, const void* a, int64_t lda, int64_t head_a,
                                      const void* w, int M, int N, int K, int heads, hipStream_t stream) {
   PAE_REQUIRE(M >= 0 && N > 0 && K > 0 && heads > 0 && heads <= 65535, "heads_product_few: bad sizes M=%d N=%d K=%d heads=%d", M, N,
               K, heads);
   if (M == 0) return 0;
+  if (K % 8 == 0 && lda % 8 == 0 && head_a % 8 == 0 && (uintptr_t)a % 16 == 0 && (uintptr_t)w % 16 == 0) {
+#define HEADS_VEC(L)                                                                                                      \
+  heads_product_few_vec_kernel<L><<<dim3((N + 4 * (64 / L) - 1) / (4 * (64 / L)), heads), 256, 0, stream>>>(               \
+      (bf16_t*)out, ldc, head_c, (const bf16_t*)a, lda, head_a, (const bf16_t*)w, M, N, K)
+    if (K <= 64) HEADS_VEC(8);
+    else if (K <= 128) HEADS_VEC(16);
+    else if (K <= 256) HEADS_VEC(32);
+    else HEADS_VEC(64);
+#undef HEADS_VEC
+    return pae_check_launch("heads_product_few");
+  }
   heads_product_few_kernel<<<dim3((N + 3) / 4, heads), 256, 0, stream>>>((bf16_t*)out, ldc, head_c, (const bf16_t*)a, lda, head_a,
                                                                        (const bf16_t*)w, M, N, K);
   return pae_check_launch("heads_product_few");

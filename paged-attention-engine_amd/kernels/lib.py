@@ -989,7 +989,13 @@ def gemm_plain_heads(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor) -> Non
                                             w.stride(0), None, 0, M, N, K, B, _stream()))
 
 
-HEADS_FEW_MAX_ROWS = 16
+HEADS_FEW_MAX_ROWS = 16       # rows up to which the few-row kernel is ahead, reading a number at a time ...
+HEADS_FEW_MAX_ROWS_VEC = 64   # ... and eight at a time (inner size and strides in multiples of eight)
+
+
+def _heads_few_rows(a: torch.Tensor) -> int:
+    eights = a.shape[2] % 8 == 0 and a.stride(0) % 8 == 0 and a.stride(1) % 8 == 0 and a.data_ptr() % 16 == 0
+    return HEADS_FEW_MAX_ROWS_VEC if eights else HEADS_FEW_MAX_ROWS
 
 
 def heads_product(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor,
@@ -997,11 +1003,11 @@ def heads_product(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor,
     """out[:, h, :] = a[:, h, :] @ w[h]^T for every head h (shapes as for `gemm_plain_heads`); `w_kn` [B, K, N] is
     the same weights the other way round (the platform's batched product takes them so; None: turned round here).  bfloat16 with
     more rows than the few-row kernels take goes to the platform's batched matrix product, as the plain
-    products of that many rows do; bfloat16 with up to 16 rows to a kernel that streams the weights once;
+    products of that many rows do; bfloat16 with a few rows to a kernel that streams the weights;
     everything else to the plain product's batched entry."""
-    if a.dtype == torch.bfloat16 and 0 < a.shape[0] <= HEADS_FEW_MAX_ROWS:
-        # a few rows: one wavefront per (head, output feature), the weights read once (every wavefront reads all rows
-        # of its head: at 64 rows that costs more than the plain kernel's tiles, measured)
+    if a.dtype == torch.bfloat16 and 0 < a.shape[0] <= _heads_few_rows(a):
+        # a few rows: a wavefront or a part of one per (head, output feature), eight rows' sums at a time (measured with
+        # 12 heads, 128 x 512: 64 rows 23 us against the plain kernel's 56; a number a load it loses from 16 rows on)
         _not_while_recording("heads_product")
         _gpu(out, a, w)
         M, B, K_ = a.shape

@@ -78,6 +78,14 @@ class PositionSpec(PartSpec):
 
 
 @dataclass(frozen=True)
+class QueryTemperature:
+    """Queries grow with their position: at position p they are multiplied by 1 + coef ln(floor((p + 1) / every) + 1)."""
+
+    coef: float
+    every: int
+
+
+@dataclass(frozen=True)
 class MixerSpec(PartSpec):
     """Causal attention over the paged cache with grouped key/value heads.
 
@@ -113,6 +121,13 @@ class MixerSpec(PartSpec):
     qk_norm_eps: float = 1e-6
     q_norm_name: str = "q_norm.weight"
     k_norm_name: str = "k_norm.weight"
+    temperature: Optional[QueryTemperature] = None
+    # values shared along the layers: "source": this layer's values are what the layers with "mixed" add to their own,
+    # v <- (1 - share) v + share v_source for the same token, share the tensor `value_mix_name` (shape []) of the layer
+    # that mixes; the mixed values are what is cached
+    value_mix: Optional[str] = None
+    value_mix_name: str = "vmix"
+    head_gate_name: Optional[str] = None  # a projection W_g [heads, hidden] of the mixer's input: head j *= sigmoid(W_g x)_j before W_o
     # and some others' (a spec with any of these runs the mixer's convolution path):
     # "head" as `qk_norm`: every query and key head divided by its own root mean square, no weight
     mask: str = "window"                 # "chunk": `window` is a chunk length, position p sees keys from p - p % window on
@@ -132,7 +147,8 @@ class MixerSpec(PartSpec):
         """The reference's attention and nothing more, with heads in multiples of 16 up to 256: what the kernels of
         the first path compute (any other head size takes the path for value widths, caps and sinks)."""
         return (self.value_dim in (None, self.head_dim) and self.softcap is None and not self.sinks
-                and self.fixed_sink is None and self.qk_norm is None and not self.convolved and self.head_dim % 16 == 0 and 16 <= self.head_dim <= 256)
+                and self.fixed_sink is None and self.qk_norm is None and self.temperature is None and self.value_mix is None
+                and self.head_gate_name is None and not self.convolved and self.head_dim % 16 == 0 and 16 <= self.head_dim <= 256)
 
     @property
     def convolved(self) -> bool:
@@ -314,6 +330,16 @@ class SideBySideSpec(PartSpec):
 
 
 @dataclass(frozen=True)
+class SharedExpertSpec:
+    """An expert that every token uses, of the same form as the routed ones and a width of its own; its output is
+    multiplied by sigmoid(W_sg h), one number per token.  Its tensors lie below `prefix` of the feed-forward's own."""
+
+    intermediate_size: int
+    prefix: str = "shared."
+    gate_name: str = "sg"   # W_sg [1, hidden]
+
+
+@dataclass(frozen=True)
 class ExpertsSpec(PartSpec):
     """A feed-forward of `num_experts` small gated experts W_down (act(W_gate h) * (W_up h)) of which a token
     uses `top`: router scores are the softmax of W_router h over all experts (float32); the experts form
@@ -332,6 +358,9 @@ class ExpertsSpec(PartSpec):
     router_name: str = "router"
     choice_bias_name: Optional[str] = None  # a tensor [experts] added to the scores where experts are chosen (the
                                             # weights stay the scores themselves); None: no such tensor
+    router_bias_name: Optional[str] = None  # a tensor [experts] added to the router's logits
+    weights_over: str = "all"   # "chosen": the weights are the softmax over the chosen logits alone (one group, no choice bias)
+    shared: Optional[SharedExpertSpec] = None
     expert_prefix: str = "e"   # expert j's tensors lie below <expert_prefix><j>.
     gate_name: str = "gate"
     up_name: str = "up"
@@ -381,6 +410,8 @@ class FeedForwardSpec(PartSpec):
     up_name: str = "up_proj"
     down_name: str = "down_proj"
     weight_suffix: str = ".weight"
+    bias: bool = False           # kind "dense": both products add a stored bias
+    bias_suffix: str = ".bias"
 
 
 @dataclass(frozen=True)
@@ -455,6 +486,8 @@ class ModelPlan:
     streams: int = 1                        # copies the residual stream is kept in (blocks of arrangement "hyper")
     pair_embedding: Optional[PairEmbeddingSpec] = None  # a hashed table of token pairs added to the embedding
     position_table_name: Optional[str] = None  # a learned row per position [max_positions, hidden], added unscaled
+    # b: sin(p b^(-2i/hidden)) and cos of the same are added to features 2i and 2i + 1 of the embedding at position p
+    sinusoid_base: Optional[float] = None
     extra: Mapping[str, Any] = field(default_factory=dict)
 
     def __post_init__(self) -> None:
@@ -474,6 +507,10 @@ class ModelPlan:
                 raise ConfigError(f"layer {i}: only the arrangement 'hyper' keeps several copies of the stream")
         if self.position_table_name is not None and not self.max_positions:
             raise ConfigError("a table of learned positions needs max_positions, its number of rows")
+        if self.sinusoid_base is not None and not self.sinusoid_base > 0:
+            raise ConfigError(f"sinusoid_base must be positive, got {self.sinusoid_base}")
+        if self.sinusoid_base is not None and (self.position_table_name is not None or self.pair_embedding is not None):
+            raise ConfigError("sinusoids of the position go with a plain embedding, not with a second table added to it")
         if self.schedule and self.schedule[0].add_embedding:
             raise ConfigError("the first stop of the schedule cannot add the embedding's output again")
         if self.logit_softcap is not None and not self.logit_softcap > 0:

@@ -119,12 +119,13 @@ int pae_qk_norm_rotate_store(int dtype, void* qkv, int64_t row_stride, int num_t
                              const void* q_w, const void* k_w, int w_is_f32, float eps, int rot, int interleaved,
                              const float* cos_sin, float magnitude, const int* positions, const int* tok_seq,
                              const int* block_tables, int max_blocks, int bs, void* k_cache, void* v_cache, int write_kv,
-                             int per_head, hipStream_t stream);
+                             int per_head, float temp_coef, int temp_every, const void* v_first,
+                             int64_t v_first_stride, float v_share, hipStream_t stream);
 // blocks that normalise a branch's output: see branch_norm.hip
 int pae_rows_from_residual(int dtype, void* out, const float* residual, int64_t n, hipStream_t stream);
 int pae_norm_scale_add(int dtype, float* residual, const void* y, int parts, int64_t part_stride, const void* weight,
                        int w_is_f32, float eps, float scale, void* next, int num_rows, int hidden, hipStream_t stream);
-int pae_activation(int dtype, void* x, int64_t n, int kind, hipStream_t stream);
+int pae_activation(int dtype, void* x, int64_t n, int kind, const void* bias, int b_is_f32, int width, hipStream_t stream);
 // the gated delta rule over a step's projected rows: see delta_rule.hip
 int pae_delta_rule_step(int dtype, const void* proj, int64_t row_stride, int num_tokens, int num_seqs, const int* tok_seq,
                         const int* positions, const int* seq_runs, const int* slots, const float* conv_w,
@@ -183,13 +184,17 @@ int pae_norm_join_conv(int dtype, float* residual, const void* y, int parts, int
 // a learned row per position added to the embedding; a layer's columns of a second token table: see token_inputs.hip
 int pae_embedding_positions(int dtype, float* out, const void* table, const int* ids, const void* rows,
                             const int* positions, int num_tokens, int hidden, int vocab, float scale, hipStream_t stream);
+// sines and cosines of a token's position added to its embedding row: see token_inputs.hip
+int pae_embedding_sinusoids(int dtype, float* out, const void* table, const int* ids, const double* turns,
+                            const int* positions, int num_tokens, int hidden, int vocab, float scale, hipStream_t stream);
 int pae_token_gate(int dtype, void* out, const void* gate, int64_t gate_stride, const void* columns, const int* ids,
                    int num_tokens, int dim, int kind, hipStream_t stream);
 // float32 sums of a few output features from rows of either type: see moe.hip
 int pae_project_f32(int dtype, float* out, int64_t ldo, const void* A, int64_t lda, const void* W, const void* bias,
                     int b_is_f32, int M, int N, int K, hipStream_t stream);
 int pae_moe_route(const float* logits, int num_tokens, int experts, int groups, int keep, int top, float scale,
-                  const float* choice_bias, int* chosen, float* weights, hipStream_t stream);
+                  const float* choice_bias, int64_t ldz, int among_chosen, int shared_pieces, int* chosen, float* weights,
+                  hipStream_t stream);
 int pae_moe_gate_up(int dtype, void* act, const void* x, int64_t ldx, const void* gate_w, const void* up_w,
                     const int* chosen, int num_tokens, int top, int hidden, int inter, int act_kind, hipStream_t stream);
 int pae_moe_tile_rows(int pairs);
@@ -209,15 +214,18 @@ int pae_attn_prefill_bf16(void* out, int64_t out_stride, const void* q, int64_t 
                           const void* v_cache, const int* tiles, int num_tiles, const int* positions,
                           const int* block_tables, int max_blocks, int bs, int nh, int nkv, int hd, float scale,
                           int window, hipStream_t stream);
-// the two above with capped scores (cap > 0: s <- cap tanh(s / cap)) and per-head sinks (float32 [nh] or null)
+// the two above with capped scores (cap > 0: s <- cap tanh(s / cap)), per-head sinks (float32 [nh] or null) and a gate
+// of one number a head (`head_gate` bfloat16 rows [token][nh], or null: out *= sigmoid(head_gate))
 int pae_attn_decode_capped_bf16(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* k_cache,
                                 const void* v_cache, const int* dec_work, int num_dec, const int* block_tables,
                                 int max_blocks, int bs, int nh, int nkv, int hd, float scale, int window, float cap,
-                                const float* sinks, void* part_acc, void* part_ml, hipStream_t stream);
+                                const float* sinks, const void* head_gate, int64_t head_gate_stride, void* part_acc,
+                                void* part_ml, hipStream_t stream);
 int pae_attn_prefill_capped_bf16(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* k_cache,
                                  const void* v_cache, const int* tiles, int num_tiles, const int* positions,
                                  const int* block_tables, int max_blocks, int bs, int nh, int nkv, int hd, float scale,
-                                 int window, float cap, const float* sinks, hipStream_t stream);
+                                 int window, float cap, const float* sinks, const void* head_gate,
+                                 int64_t head_gate_stride, hipStream_t stream);
 // the two with the window read as a chunk length (`chunked`), a bias by distance (`slopes` float32 [nh] or null:
 // score -= slopes[h] (position - key)) and a gate on the output (`gate` bfloat16 rows [token][nh * hd] or null)
 int pae_attn_decode_biased_bf16(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* k_cache,

@@ -176,7 +176,8 @@ __global__ void attn_decode_merge_kernel(bf16_t* __restrict__ out, int64_t out_s
                                          const float* __restrict__ part_acc, const float* __restrict__ part_ml,
                                          int max_splits, const int4* __restrict__ dec_work, int nh, int nkv,
                                          int window, const float* __restrict__ sinks, int chunked,
-                                         const bf16_t* __restrict__ gate, int64_t gate_stride) {
+                                         const bf16_t* __restrict__ gate, int64_t gate_stride,
+                                         const bf16_t* __restrict__ head_gate, int64_t head_gate_stride) {
   // blockDim = (items rounded up to wavefronts, G): the splits are dealt out to G groups of threads,
   // whose loads are all in flight together; group 0 then adds the groups' sums in group order.
   extern __shared__ float s_merge[];  // [G - 1][items][6]: four sums, maximum, sum of weights
@@ -228,7 +229,9 @@ __global__ void attn_decode_merge_kernel(bf16_t* __restrict__ out, int64_t out_s
     a = a * f_old;
     l = l * f_old + exp2f(sink - m_new);
   }
-  const float inv = 1.0f / l;
+  float inv = 1.0f / l;
+  if (head_gate)  // one number a token and head
+    inv /= 1.0f + expf(-__bfloat162float(head_gate[(int64_t)tok * head_gate_stride + kvh * g + c]));
   s16x4 w;
   if (gate) {
     const bf16_t* gt = gate + (int64_t)tok * gate_stride + (int64_t)(kvh * g + c) * HD + d;
@@ -615,11 +618,13 @@ static int attn_decode_any(void* out, int64_t out_stride, const void* q, int64_t
                                     const void* k_cache, const void* v_cache, const int* dec_work, int num_dec,
                                     const int* block_tables, int max_blocks, int bs, int nh, int nkv, int hd, float scale, int window,
                                     float cap, const float* sinks, void* part_acc, void* part_ml, bool biased, int chunked,
-                                    const float* slopes, const void* gate, int64_t gate_stride, hipStream_t stream) {
+                                    const float* slopes, const void* gate, int64_t gate_stride, const void* head_gate,
+                                    int64_t head_gate_stride, hipStream_t stream) {
   if (int rc = check_common("attn_decode", nh, nkv, hd, bs, max_blocks, window)) return rc;
   PAE_REQUIRE(!biased || cap == 0.f, "attn_decode: a bias by distance and a score cap together are not built");
   PAE_REQUIRE(biased || (!chunked && !slopes && !gate), "attn_decode: chunks, slopes and gates belong to the biased kernels");
   PAE_REQUIRE(!gate || gate_stride >= (int64_t)nh * hd, "attn_decode: gate row stride %lld too small", (long long)gate_stride);
+  PAE_REQUIRE(!head_gate || head_gate_stride >= nh, "attn_decode: head gate row stride %lld too small", (long long)head_gate_stride);
   PAE_REQUIRE(num_dec <= 65535 && nkv <= 65535, "attn_decode: grid too large");
   if (num_dec <= 0) return 0;
   const int split_len = 64 * DECODE_TPW;
@@ -652,7 +657,7 @@ static int attn_decode_any(void* out, int64_t out_stride, const void* q, int64_t
   }                                                                                                         \
   attn_decode_merge_kernel<HD, DECODE_TPW><<<merge_grid, dim3(merge_x, merge_groups), merge_lds, stream>>>( \
       (bf16_t*)out, out_stride, (const float*)part_acc, (const float*)part_ml, max_splits, (const int4*)dec_work, \
-      nh, nkv, window, sinks, chunked, (const bf16_t*)gate, gate_stride)
+      nh, nkv, window, sinks, chunked, (const bf16_t*)gate, gate_stride, (const bf16_t*)head_gate, head_gate_stride)
   FOR_HEAD_DIM(hd, CALL)
 #undef CALL
 #undef CALL_CAPPED
@@ -662,9 +667,11 @@ static int attn_decode_any(void* out, int64_t out_stride, const void* q, int64_t
 extern "C" int pae_attn_decode_capped_bf16(void* out, int64_t out_stride, const void* q, int64_t q_stride,
                                     const void* k_cache, const void* v_cache, const int* dec_work, int num_dec,
                                     const int* block_tables, int max_blocks, int bs, int nh, int nkv, int hd, float scale, int window,
-                                    float cap, const float* sinks, void* part_acc, void* part_ml, hipStream_t stream) {
+                                    float cap, const float* sinks, const void* head_gate, int64_t head_gate_stride,
+                                    void* part_acc, void* part_ml, hipStream_t stream) {
   return attn_decode_any(out, out_stride, q, q_stride, k_cache, v_cache, dec_work, num_dec, block_tables, max_blocks, bs, nh,
-                         nkv, hd, scale, window, cap, sinks, part_acc, part_ml, false, 0, nullptr, nullptr, 0, stream);
+                         nkv, hd, scale, window, cap, sinks, part_acc, part_ml, false, 0, nullptr, nullptr, 0, head_gate,
+                         head_gate_stride, stream);
 }
 
 // `chunked`: the window is a chunk length; `slopes` (float32 [nh] or null): score -= slopes[h] (position - key);
@@ -676,7 +683,7 @@ extern "C" int pae_attn_decode_biased_bf16(void* out, int64_t out_stride, const 
                                     void* part_ml, hipStream_t stream) {
   return attn_decode_any(out, out_stride, q, q_stride, k_cache, v_cache, dec_work, num_dec, block_tables, max_blocks, bs, nh,
                          nkv, hd, scale, window, 0.f, nullptr, part_acc, part_ml, true, chunked, slopes, gate, gate_stride,
-                         stream);
+                         nullptr, 0, stream);
 }
 
 extern "C" int pae_attn_decode_bf16(void* out, int64_t out_stride, const void* q, int64_t q_stride,
@@ -684,7 +691,7 @@ extern "C" int pae_attn_decode_bf16(void* out, int64_t out_stride, const void* q
                                     const int* block_tables, int max_blocks, int bs, int nh, int nkv, int hd, float scale, int window,
                                     void* part_acc, void* part_ml, hipStream_t stream) {
   return pae_attn_decode_capped_bf16(out, out_stride, q, q_stride, k_cache, v_cache, dec_work, num_dec, block_tables,
-                                     max_blocks, bs, nh, nkv, hd, scale, window, 0.f, nullptr, part_acc, part_ml, stream);
+                                     max_blocks, bs, nh, nkv, hd, scale, window, 0.f, nullptr, nullptr, 0, part_acc, part_ml, stream);
 }
 
 // tiles[t] = (table row of the sequence, first flat token, number of tokens <= 64), heaviest runs
@@ -694,12 +701,15 @@ static int attn_prefill_any(void* out, int64_t out_stride, const void* q, int64_
                                           int num_tiles, const int* positions, const int* block_tables,
                                           int max_blocks, int bs, int nh, int nkv, int hd, float scale, int window,
                                           float cap, const float* sinks, bool biased, int chunked, const float* slopes,
-                                          const void* gate, int64_t gate_stride, hipStream_t stream) {
+                                          const void* gate, int64_t gate_stride, const void* head_gate,
+                                          int64_t head_gate_stride, hipStream_t stream) {
   if (int rc = check_common("attn_prefill", nh, nkv, hd, bs, max_blocks, window)) return rc;
   PAE_REQUIRE(!biased || cap == 0.f, "attn_prefill: a bias by distance and a score cap together are not built");
   PAE_REQUIRE(!biased || !slopes || scale > 0.f, "attn_prefill: a bias by distance needs a positive scale");
   PAE_REQUIRE(biased || (!chunked && !slopes && !gate), "attn_prefill: chunks, slopes and gates belong to the biased kernels");
   PAE_REQUIRE(!gate || gate_stride >= (int64_t)nh * hd, "attn_prefill: gate row stride %lld too small", (long long)gate_stride);
+  PAE_REQUIRE(!head_gate || (!biased && head_gate_stride >= nh), "attn_prefill: head gate row stride %lld too small, or a biased kernel",
+              (long long)head_gate_stride);
   PAE_REQUIRE(num_tiles <= 65535, "attn_prefill: %d runs exceed the grid", num_tiles);
   if (num_tiles <= 0) return 0;
   const float scale_log2 = scale * LOG2E;
@@ -714,7 +724,7 @@ static int attn_prefill_any(void* out, int64_t out_stride, const void* q, int64_
   attn_prefill_split_kernel<HD, CT, BS, CAPPED, BIASED><<<dim3(nh, num_tiles, 4 / CT), 256, 0, stream>>>(      \
       (bf16_t*)out, out_stride, (const bf16_t*)q, q_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,    \
       tiles, positions, block_tables, max_blocks, bs, nh, nkv, scale_log2, window, cap_over_scale,             \
-      scale_over_cap, sinks, chunked, slopes, slopes ? 1.0f / scale : 0.f, (const bf16_t*)gate, gate_stride, nullptr, 0)
+      scale_over_cap, sinks, chunked, slopes, slopes ? 1.0f / scale : 0.f, (const bf16_t*)gate, gate_stride, (const bf16_t*)head_gate, head_gate_stride)
 #define LAUNCH_CT(HD, CT, BS)                  \
   if (biased) {                                \
     LAUNCH_CAPPED(HD, CT, BS, false, true);    \
@@ -747,9 +757,11 @@ extern "C" int pae_attn_prefill_capped_bf16(void* out, int64_t out_stride, const
                                           const void* k_cache, const void* v_cache, const int* tiles,
                                           int num_tiles, const int* positions, const int* block_tables,
                                           int max_blocks, int bs, int nh, int nkv, int hd, float scale, int window,
-                                          float cap, const float* sinks, hipStream_t stream) {
+                                          float cap, const float* sinks, const void* head_gate, int64_t head_gate_stride,
+                                          hipStream_t stream) {
   return attn_prefill_any(out, out_stride, q, q_stride, k_cache, v_cache, tiles, num_tiles, positions, block_tables,
-                          max_blocks, bs, nh, nkv, hd, scale, window, cap, sinks, false, 0, nullptr, nullptr, 0, stream);
+                          max_blocks, bs, nh, nkv, hd, scale, window, cap, sinks, false, 0, nullptr, nullptr, 0, head_gate,
+                          head_gate_stride, stream);
 }
 
 extern "C" int pae_attn_prefill_biased_bf16(void* out, int64_t out_stride, const void* q, int64_t q_stride,
@@ -760,7 +772,7 @@ extern "C" int pae_attn_prefill_biased_bf16(void* out, int64_t out_stride, const
                                           hipStream_t stream) {
   return attn_prefill_any(out, out_stride, q, q_stride, k_cache, v_cache, tiles, num_tiles, positions, block_tables,
                           max_blocks, bs, nh, nkv, hd, scale, window, 0.f, nullptr, true, chunked, slopes, gate, gate_stride,
-                          stream);
+                          nullptr, 0, stream);
 }
 
 extern "C" int pae_attn_prefill_bf16(void* out, int64_t out_stride, const void* q, int64_t q_stride,
@@ -768,7 +780,7 @@ extern "C" int pae_attn_prefill_bf16(void* out, int64_t out_stride, const void* 
                                      const int* positions, const int* block_tables, int max_blocks, int bs, int nh,
                                      int nkv, int hd, float scale, int window, hipStream_t stream) {
   return pae_attn_prefill_capped_bf16(out, out_stride, q, q_stride, k_cache, v_cache, tiles, num_tiles, positions,
-                                      block_tables, max_blocks, bs, nh, nkv, hd, scale, window, 0.f, nullptr, stream);
+                                      block_tables, max_blocks, bs, nh, nkv, hd, scale, window, 0.f, nullptr, nullptr, 0, stream);
 }
 
 // Key widths `hd` (multiples of 32 up to 256) built for values `vd` wide: the smallest that holds `width` features, or 0.

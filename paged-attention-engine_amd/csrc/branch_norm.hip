@@ -152,38 +152,50 @@ extern "C" int pae_norm_scale_add(int dtype, float* residual, const void* y, int
 }
 
 template <typename T>
-__global__ void activation_kernel(T* __restrict__ x, int64_t n, int kind) {
+__global__ void activation_kernel(T* __restrict__ x, int64_t n, int kind, const void* __restrict__ bias, int b_is_f32,
+                                  int width) {
   const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i < n) x[i] = from_f32<T>(act_of(to_f32(x[i]), kind));
+  if (i < n) x[i] = from_f32<T>(act_of(to_f32(x[i]) + (bias ? load_param(bias, b_is_f32, i % width) : 0.f), kind));
 }
 
-// eight bfloat16 numbers a thread (one 16-byte load and store), for sizes that are multiples of eight
-__global__ void activation_bf16x8_kernel(uint4* __restrict__ x, int64_t nvec, int kind) {
+// eight bfloat16 numbers a thread (one 16-byte load and store), for sizes (and widths, with a bias) that are
+// multiples of eight
+__global__ void activation_bf16x8_kernel(uint4* __restrict__ x, int64_t nvec, int kind, const void* __restrict__ bias,
+                                         int b_is_f32, int width) {
   const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= nvec) return;
   uint4 v = x[i];
   unsigned* w = reinterpret_cast<unsigned*>(&v);
+  float b[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+  if (bias) {
+    const int first = (int)(8 * i % width);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) b[j] = load_param(bias, b_is_f32, first + j);
+  }
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
-    const bf16_t lo = __float2bfloat16(act_of(__uint_as_float(w[j] << 16), kind));
-    const bf16_t hi = __float2bfloat16(act_of(__uint_as_float(w[j] & 0xffff0000u), kind));
+    const bf16_t lo = __float2bfloat16(act_of(__uint_as_float(w[j] << 16) + b[2 * j], kind));
+    const bf16_t hi = __float2bfloat16(act_of(__uint_as_float(w[j] & 0xffff0000u) + b[2 * j + 1], kind));
     w[j] = (unsigned)*reinterpret_cast<const unsigned short*>(&lo) | ((unsigned)*reinterpret_cast<const unsigned short*>(&hi) << 16);
   }
   x[i] = v;
 }
 
-extern "C" int pae_activation(int dtype, void* x, int64_t n, int kind, hipStream_t stream) {
-  PAE_REQUIRE(kind >= 0 && kind <= 2, "activation: unknown kind %d", kind);
+// x <- act(x + bias): rows of `width` numbers, bias (or null) one number per column
+extern "C" int pae_activation(int dtype, void* x, int64_t n, int kind, const void* bias, int b_is_f32, int width,
+                              hipStream_t stream) {
+  PAE_REQUIRE(!bias || (width > 0 && n % width == 0), "activation: %lld numbers are no rows of %d", (long long)n, width);
+  PAE_REQUIRE(kind >= 0 && kind <= PAE_LAST_ACTIVATION, "activation: unknown kind %d", kind);
   if (n <= 0) return 0;
-  if (dtype == PAE_BF16 && n % 8 == 0 && (uintptr_t)x % 16 == 0) {
-    activation_bf16x8_kernel<<<(unsigned)((n / 8 + 255) / 256), 256, 0, stream>>>((uint4*)x, n / 8, kind);
+  if (dtype == PAE_BF16 && n % 8 == 0 && (uintptr_t)x % 16 == 0 && (!bias || width % 8 == 0)) {
+    activation_bf16x8_kernel<<<(unsigned)((n / 8 + 255) / 256), 256, 0, stream>>>((uint4*)x, n / 8, kind, bias, b_is_f32, width);
     return pae_check_launch("activation");
   }
   const unsigned blocks = (unsigned)((n + 255) / 256);
   if (dtype == PAE_F32)
-    activation_kernel<float><<<blocks, 256, 0, stream>>>((float*)x, n, kind);
+    activation_kernel<float><<<blocks, 256, 0, stream>>>((float*)x, n, kind, bias, b_is_f32, width);
   else if (dtype == PAE_BF16)
-    activation_kernel<bf16_t><<<blocks, 256, 0, stream>>>((bf16_t*)x, n, kind);
+    activation_kernel<bf16_t><<<blocks, 256, 0, stream>>>((bf16_t*)x, n, kind, bias, b_is_f32, width);
   else
     return pae_fail("activation: unknown dtype code %d", dtype);
   return pae_check_launch("activation");

@@ -557,7 +557,7 @@ extern "C" int pae_gated_act(int dtype, void* out, const void* x, int num_tokens
                              hipStream_t stream) {
   PAE_REQUIRE(num_tokens >= 0 && inter > 0, "gated_act: bad sizes T=%d I=%d", num_tokens, inter);
   PAE_REQUIRE(block >= 0 && (block == 0 || inter % block == 0), "gated_act: blocks of %d do not divide %d", block, inter);
-  PAE_REQUIRE(kind >= 0 && kind <= 2, "gated_act: unknown activation code %d", kind);
+  PAE_REQUIRE(kind >= 0 && kind <= PAE_LAST_ACTIVATION, "gated_act: unknown activation code %d", kind);
   const int64_t total = (int64_t)num_tokens * inter;
   if (total == 0) return 0;
   const unsigned blocks = (unsigned)((total + 255) / 256);

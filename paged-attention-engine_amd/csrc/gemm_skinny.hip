@@ -568,11 +568,11 @@ extern "C" int pae_gemm_skinny(int epilogue, void* out, int64_t ldc, const void*
 }
 
 // out[M, N] = bfloat16(act(A W^T + bias)): the plain epilogue with an activation (0 gelu by erf, 1 gelu by tanh,
-// 2 silu) on the finished sums, in float32, before they are rounded.
+// 2 silu, 3 relu squared) on the finished sums, in float32, before they are rounded.
 extern "C" int pae_gemm_skinny_act(void* out, int64_t ldc, const void* A, int64_t lda, const void* W, const void* bias,
                                    int b_is_f32, int M, int N, int K, int splits, float* ticket_parts,
                                    int* ticket_counters, int act, hipStream_t stream) {
-  PAE_REQUIRE(act >= 0 && act <= 2, "gemm_skinny_act: unknown activation %d", act);
+  PAE_REQUIRE(act >= 0 && act <= PAE_LAST_ACTIVATION, "gemm_skinny_act: unknown activation %d", act);
   const SkinnyNorm norm{nullptr, 0, 0.f, nullptr, 0, nullptr, 0, act + 1, nullptr};
   return launch_skinny(EPI_BF16, out, ldc, A, lda, W, bias, b_is_f32, M, N, K, splits, 0, SkinnyRope{},
                        SkinnyTickets{ticket_parts, ticket_counters}, norm, stream);
@@ -582,7 +582,7 @@ extern "C" int pae_gemm_skinny_act(void* out, int64_t ldc, const void* A, int64_
 // activation by code: out[M, N / 2] = act(gate) * up on the float32 sums.
 extern "C" int pae_gemm_skinny_gated(void* out, int64_t ldc, const void* A, int64_t lda, const void* W, int M, int N, int K,
                                      int splits, float* ticket_parts, int* ticket_counters, int act, hipStream_t stream) {
-  PAE_REQUIRE(act >= 0 && act <= 2, "gemm_skinny_gated: unknown activation %d", act);
+  PAE_REQUIRE(act >= 0 && act <= PAE_LAST_ACTIVATION, "gemm_skinny_gated: unknown activation %d", act);
   PAE_REQUIRE(N % 16 == 0 && ldc % 4 == 0, "gemm_skinny_gated: gated epilogue needs N %% 16 == 0, got %d", N);
   const SkinnyNorm norm{nullptr, 0, 0.f, nullptr, 0, nullptr, 0, act + 1, nullptr};
   return launch_skinny(EPI_SWIGLU, out, ldc, A, lda, W, nullptr, 0, M, N, K, splits, 0, SkinnyRope{},

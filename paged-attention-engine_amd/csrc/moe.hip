@@ -7,7 +7,11 @@
 //                   `keep` best groups can be chosen; the `top` largest scores among those are chosen,
 //                   and their weights are the scores times `scale` (not renormalised).  Of equal
 //                   scores the lower index wins.  With a `choice_bias` [E], experts and groups are compared
-//                   by score + bias, while the weights stay the scores themselves.  One wavefront a token.
+//                   by score + bias, while the weights stay the scores themselves.  With `among_chosen`
+//                   instead, experts are compared by their logits and the weights are the softmax over
+//                   the chosen logits alone, times `scale`.  Experts that every token uses are `shared_pieces`
+//                   more entries behind the chosen ones, experts E, E + 1, ..., each weighted by the sigmoid
+//                   of the logit behind the experts' own.  One wavefront a token.
 //   moe_gate_up     for every (token, chosen expert): act(W_gate x) * (W_up x), rounded to the activation type
 //   moe_down        for every token: sum over its chosen experts of weight * W_down act, float32
 //
@@ -89,6 +93,7 @@ extern "C" int pae_project_f32(int dtype, float* out, int64_t ldo, const void* A
 
 __global__ __launch_bounds__(PAE_WAVE) void moe_route_kernel(const float* __restrict__ logits, int E, int groups, int keep,
                                                              int top, float scale, const float* __restrict__ choice_bias,
+                                                             int64_t ldz, int among_chosen, int shared_pieces,
                                                              int* __restrict__ chosen, float* __restrict__ weights) {
   extern __shared__ float lds[];  // [E] scores, [groups] group scores, and with a bias [E] what experts are compared by
   float* score = lds;
@@ -96,13 +101,14 @@ __global__ __launch_bounds__(PAE_WAVE) void moe_route_kernel(const float* __rest
   float* rank = choice_bias ? group_score + groups : score;
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x;
-  const float* z = logits + t * E;
+  const float* z = logits + t * ldz;
+  const int places = top + shared_pieces;
   float top_z = -INFINITY;
   for (int e = lane; e < E; e += PAE_WAVE) top_z = fmaxf(top_z, z[e]);
   top_z = wave_max(top_z);
   float sum = 0.f;
   for (int e = lane; e < E; e += PAE_WAVE) {
-    const float p = expf(z[e] - top_z);
+    const float p = among_chosen ? z[e] : expf(z[e] - top_z);
     score[e] = p;
     sum += p;
   }
@@ -132,6 +138,7 @@ __global__ __launch_bounds__(PAE_WAVE) void moe_route_kernel(const float* __rest
       if (before < keep) mine[j] = rank[e];
     }
   }
+  float first = 0.f, total = 0.f;  // among_chosen: the largest chosen logit, and the sum of exponentials against it
   for (int r = 0; r < top; ++r) {
     float best = -INFINITY;
     int at = 0x7fffffff;
@@ -149,18 +156,32 @@ __global__ __launch_bounds__(PAE_WAVE) void moe_route_kernel(const float* __rest
         at = other_at;
       }
     }
+    if (at >= E) at = 0;  // no logit compares (not a number): an index that exists
+    if (r == 0) first = best;
+    if (among_chosen) total += expf(best - first);
     if (lane == 0) {
-      chosen[t * top + r] = at;
-      weights[t * top + r] = score[at] / sum * scale;
+      chosen[t * places + r] = at;
+      weights[t * places + r] = among_chosen ? expf(best - first) : score[at] / sum * scale;
     }
 #pragma unroll
     for (int j = 0; j < MOE_MAX_PER_LANE; ++j)
       if (lane + PAE_WAVE * j == at) mine[j] = -INFINITY;
   }
+  if (lane != 0) return;
+  if (among_chosen)  // this lane's own numbers of the loop above, brought to their sum
+    for (int r = 0; r < top; ++r) weights[t * places + r] = weights[t * places + r] / total * scale;
+  for (int p = 0; p < shared_pieces; ++p) {
+    chosen[t * places + top + p] = E + p;
+    weights[t * places + top + p] = 1.0f / (1.0f + expf(-z[E]));
+  }
 }
 
 extern "C" int pae_moe_route(const float* logits, int num_tokens, int experts, int groups, int keep, int top, float scale,
-                             const float* choice_bias, int* chosen, float* weights, hipStream_t stream) {
+                             const float* choice_bias, int64_t ldz, int among_chosen, int shared_pieces, int* chosen,
+                             float* weights, hipStream_t stream) {
+  PAE_REQUIRE(ldz >= experts + (shared_pieces > 0 ? 1 : 0) && shared_pieces >= 0, "routing: rows of %lld logits for %d experts and %d shared pieces",
+              (long long)ldz, experts, shared_pieces);
+  PAE_REQUIRE(!among_chosen || (groups == 1 && !choice_bias), "routing: a softmax over the chosen logits goes with one group and no choice bias");
   PAE_REQUIRE(experts > 0 && experts <= PAE_WAVE * MOE_MAX_PER_LANE, "routing: %d experts (1..%d)", experts,
               PAE_WAVE * MOE_MAX_PER_LANE);
   PAE_REQUIRE(groups > 0 && experts % groups == 0 && keep > 0 && keep <= groups, "routing: %d groups of %d experts, %d kept",
@@ -169,7 +190,7 @@ extern "C" int pae_moe_route(const float* logits, int num_tokens, int experts, i
               keep * (experts / groups));
   if (num_tokens <= 0) return 0;
   moe_route_kernel<<<num_tokens, PAE_WAVE, (size_t)(experts + groups + (choice_bias ? experts : 0)) * sizeof(float), stream>>>(
-      logits, experts, groups, keep, top, scale, choice_bias, chosen, weights);
+      logits, experts, groups, keep, top, scale, choice_bias, ldz, among_chosen, shared_pieces, chosen, weights);
   return pae_check_launch("moe_route");
 }
 

@@ -9,6 +9,10 @@
 // token's angles: pair i is (2i, 2i + 1) with `interleaved`, (i, i + rot / 2) without, and
 //   (u, v) -> (u c - v s, v c + u s),  c = magnitude * cos(angle_i), s = magnitude * sin(angle_i)
 // (a magnitude other than 1 is what frequency-scaled rotations multiply their tables by).
+// Two things more, each switched by a parameter: a temperature on the queries, every query head times
+// 1 + temp_coef ln(floor((p + 1) / temp_every) + 1) at position p (temp_every 0: none); and values mixed with those of
+// another layer, v <- (1 - v_share) v + v_share v_first, where row t of `v_first` holds that layer's values of the same
+// token (null: none); the mixed values are what the cache receives, the row keeps its own.
 // Statistics, weights and the rotation are float32; a value is rounded to the storage type once,
 // when it is written: queries in place, keys to [block][kv head][offset][hd], values transposed
 // within the page, [block][kv head][vd][offset].
@@ -21,7 +25,8 @@ __global__ __launch_bounds__(256) void qk_norm_rotate_store_kernel(
     const void* __restrict__ k_w, int w_is_f32, float eps, int rot, int interleaved,
     const float* __restrict__ cos_sin, float magnitude, const int* __restrict__ positions,
     const int* __restrict__ tok_seq, const int* __restrict__ block_tables, int max_blocks, int bs,
-    T* __restrict__ k_cache, T* __restrict__ v_cache, int write_kv, int per_head) {
+    T* __restrict__ k_cache, T* __restrict__ v_cache, int write_kv, int per_head, float temp_coef, int temp_every,
+    const T* __restrict__ v_first, int64_t v_first_stride, float v_share) {
   extern __shared__ float head_inv[];  // [nh + nkv] with `per_head`
   __shared__ float scratch[4];
   const int t = blockIdx.x;
@@ -65,8 +70,9 @@ __global__ __launch_bounds__(256) void qk_norm_rotate_store_kernel(
     if (per_head) return x * head_inv[j / hd] * load_param(j < nq ? q_w : k_w, w_is_f32, j % hd);
     return j < nq ? x * inv_q * load_param(q_w, w_is_f32, j) : x * inv_k * load_param(k_w, w_is_f32, j - nq);
   };
+  const float temp = temp_every > 0 ? 1.0f + temp_coef * logf((float)((pos + 1) / temp_every + 1)) : 1.0f;
   auto put = [&](int h, int i, float value) {  // head h (queries first, then keys), feature i
-    if (h < nh) row[h * hd + i] = from_f32<T>(value);
+    if (h < nh) row[h * hd + i] = from_f32<T>(value * temp);
     else k_cache[k_base + ((int64_t)(h - nh) * bs + off) * hd + i] = from_f32<T>(value);
   };
   const int half = rot / 2;
@@ -80,16 +86,18 @@ __global__ __launch_bounds__(256) void qk_norm_rotate_store_kernel(
     put(h, ib, b * c + a * s);
   }
   const int tail = hd - rot;  // features beyond the rotated ones: normalised (or copied) only
-  if (q_w || write_kv)
+  if (q_w || write_kv || temp_every > 0)
     for (int idx = threadIdx.x; idx < heads * tail; idx += 256) {
       const int h = idx / tail, i = rot + idx % tail;
-      if (h < nh && !q_w) continue;
+      if (h < nh && !q_w && temp_every <= 0) continue;
       put(h, i, at(h * hd + i));
     }
   if (!write_kv) return;
   for (int idx = threadIdx.x; idx < nkv * vd; idx += 256) {
     const int h = idx / vd, i = idx % vd;
-    v_cache[v_base + ((int64_t)h * vd + i) * bs + off] = row[nq + nk + idx];
+    T value = row[nq + nk + idx];
+    if (v_first) value = from_f32<T>((1.0f - v_share) * to_f32(value) + v_share * to_f32(v_first[(int64_t)t * v_first_stride + idx]));
+    v_cache[v_base + ((int64_t)h * vd + i) * bs + off] = value;
   }
 }
 
@@ -98,7 +106,8 @@ extern "C" int pae_qk_norm_rotate_store(int dtype, void* qkv, int64_t row_stride
                                         int rot, int interleaved, const float* cos_sin, float magnitude,
                                         const int* positions, const int* tok_seq, const int* block_tables,
                                         int max_blocks, int bs, void* k_cache, void* v_cache, int write_kv,
-                                        int per_head, hipStream_t stream) {
+                                        int per_head, float temp_coef, int temp_every, const void* v_first,
+                                        int64_t v_first_stride, float v_share, hipStream_t stream) {
   PAE_REQUIRE(nh > 0 && nkv >= 0 && hd > 0 && vd > 0, "qk_norm_rotate_store: bad head sizes nh=%d nkv=%d hd=%d vd=%d",
               nh, nkv, hd, vd);
   PAE_REQUIRE(rot >= 0 && rot <= hd && rot % 2 == 0, "qk_norm_rotate_store: %d rotated features of %d", rot, hd);
@@ -108,17 +117,22 @@ extern "C" int pae_qk_norm_rotate_store(int dtype, void* qkv, int64_t row_stride
               (long long)row_stride);
   PAE_REQUIRE(!write_kv || (nkv > 0 && bs > 0 && max_blocks > 0 && k_cache && v_cache && block_tables && tok_seq),
               "qk_norm_rotate_store: a cache write needs tables and pools");
+  PAE_REQUIRE(temp_every >= 0, "qk_norm_rotate_store: a temperature that grows every %d positions", temp_every);
+  PAE_REQUIRE(!v_first || (write_kv && v_first_stride >= (int64_t)nkv * vd), "qk_norm_rotate_store: values to mix in without a cache write, or rows of %lld",
+              (long long)v_first_stride);
   if (num_tokens <= 0) return 0;
   const size_t lds = per_head ? (size_t)(nh + nkv) * sizeof(float) : 0;
   PAE_REQUIRE(lds <= 32768, "qk_norm_rotate_store: %d heads with norms of their own", nh + nkv);
   if (dtype == PAE_F32)
     qk_norm_rotate_store_kernel<float><<<num_tokens, 256, lds, stream>>>(
         (float*)qkv, row_stride, nh, nkv, hd, vd, q_w, k_w, w_is_f32, eps, rot, interleaved, cos_sin, magnitude,
-        positions, tok_seq, block_tables, max_blocks, bs, (float*)k_cache, (float*)v_cache, write_kv, per_head);
+        positions, tok_seq, block_tables, max_blocks, bs, (float*)k_cache, (float*)v_cache, write_kv, per_head,
+        temp_coef, temp_every, (const float*)v_first, v_first_stride, v_share);
   else if (dtype == PAE_BF16)
     qk_norm_rotate_store_kernel<bf16_t><<<num_tokens, 256, lds, stream>>>(
         (bf16_t*)qkv, row_stride, nh, nkv, hd, vd, q_w, k_w, w_is_f32, eps, rot, interleaved, cos_sin, magnitude,
-        positions, tok_seq, block_tables, max_blocks, bs, (bf16_t*)k_cache, (bf16_t*)v_cache, write_kv, per_head);
+        positions, tok_seq, block_tables, max_blocks, bs, (bf16_t*)k_cache, (bf16_t*)v_cache, write_kv, per_head,
+        temp_coef, temp_every, (const bf16_t*)v_first, v_first_stride, v_share);
   else
     return pae_fail("qk_norm_rotate_store: unknown dtype code %d", dtype);
   return pae_check_launch("qk_norm_rotate_store");

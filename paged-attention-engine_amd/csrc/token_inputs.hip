@@ -2,9 +2,12 @@
 // columns of a second token table that gate a narrow product of the stream.
 //
 //   embedding_positions   out[t] = scale * table[ids[t]] + rows[positions[t]]  (float32; the position's row unscaled)
+//   embedding_sinusoids   out[t] = scale * table[ids[t]] + P(positions[t]), entry 2i of P(p) the sine and 2i + 1 the cosine
+//                         of p times the i-th frequency: `turns` holds the frequencies over 2 pi in double precision, the
+//                         angle is reduced to a fraction of a turn in double precision and rounded to float32 then
 //   token_gate            out[t][i] = T(act(gate[t][i]) * columns[ids[t]][i]): `gate` is a narrow product of the
 //                         stream, `columns` [vocab][dim] the layer's share of the second table; the activation
-//                         (0 gelu by erf, 1 gelu by tanh, 2 silu) and the product are float32, rounded once
+//                         (by code, see act_of) and the product are float32, rounded once
 #include "common.h"
 #include "api.h"
 
@@ -38,6 +41,39 @@ extern "C" int pae_embedding_positions(int dtype, float* out, const void* table,
 }
 
 template <typename T>
+__global__ void embedding_sinusoids_kernel(float* __restrict__ out, const T* __restrict__ table, const int* __restrict__ ids,
+                                           const double* __restrict__ turns, const int* __restrict__ positions, int hidden,
+                                           float scale) {
+  const int t = blockIdx.x;
+  const T* row = table + (int64_t)ids[t] * hidden;
+  const double p = (double)positions[t];
+  float* dst = out + (int64_t)t * hidden;
+  for (int i = threadIdx.x; 2 * i < hidden; i += blockDim.x) {
+    const double angle = p * turns[i];
+    float s, c;
+    sincospif(2.0f * (float)(angle - rint(angle)), &s, &c);
+    dst[2 * i] = scale * to_f32(row[2 * i]) + s;
+    if (2 * i + 1 < hidden) dst[2 * i + 1] = scale * to_f32(row[2 * i + 1]) + c;
+  }
+}
+
+extern "C" int pae_embedding_sinusoids(int dtype, float* out, const void* table, const int* ids, const double* turns,
+                                       const int* positions, int num_tokens, int hidden, int vocab, float scale,
+                                       hipStream_t stream) {
+  PAE_REQUIRE(num_tokens >= 0 && hidden > 0 && vocab > 0, "embedding with sinusoids: bad sizes T=%d H=%d V=%d", num_tokens,
+              hidden, vocab);
+  PAE_REQUIRE(table && turns && ids && positions, "embedding with sinusoids: a table, frequencies and both index lists are needed");
+  if (num_tokens == 0) return 0;
+  if (dtype == PAE_F32)
+    embedding_sinusoids_kernel<float><<<num_tokens, 256, 0, stream>>>(out, (const float*)table, ids, turns, positions, hidden, scale);
+  else if (dtype == PAE_BF16)
+    embedding_sinusoids_kernel<bf16_t><<<num_tokens, 256, 0, stream>>>(out, (const bf16_t*)table, ids, turns, positions, hidden, scale);
+  else
+    return pae_fail("embedding with sinusoids: unknown dtype code %d", dtype);
+  return pae_check_launch("embedding_sinusoids");
+}
+
+template <typename T>
 __global__ __launch_bounds__(256) void token_gate_kernel(T* __restrict__ out, const T* __restrict__ gate, int64_t gate_stride,
                                                          const T* __restrict__ columns, const int* __restrict__ ids,
                                                          int dim, int kind, int64_t total) {
@@ -51,7 +87,7 @@ __global__ __launch_bounds__(256) void token_gate_kernel(T* __restrict__ out, co
 extern "C" int pae_token_gate(int dtype, void* out, const void* gate, int64_t gate_stride, const void* columns,
                               const int* ids, int num_tokens, int dim, int kind, hipStream_t stream) {
   PAE_REQUIRE(dim > 0 && gate_stride >= dim, "token gate: %d columns in rows of %lld", dim, (long long)gate_stride);
-  PAE_REQUIRE(kind >= 0 && kind <= 2, "token gate: unknown activation code %d", kind);
+  PAE_REQUIRE(kind >= 0 && kind <= PAE_LAST_ACTIVATION, "token gate: unknown activation code %d", kind);
   if (num_tokens <= 0) return 0;
   const int64_t total = (int64_t)num_tokens * dim;
   const unsigned blocks = (unsigned)((total + 255) / 256);

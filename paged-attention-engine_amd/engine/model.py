@@ -11,6 +11,7 @@ reference's proof that a step is one pass (:180-186,338).
 
 from __future__ import annotations
 
+import math
 from typing import Dict, List, Mapping, Optional, Tuple
 
 import torch
@@ -92,6 +93,10 @@ class Model:
         self.position_table = None
         if plan.position_table_name is not None:
             self.position_table = weights[plan.position_table_name].to(device=self.device, dtype=self.dtype).contiguous()
+        self.turns = None
+        if plan.sinusoid_base is not None:  # the positions' frequencies in turns a position, in double precision
+            i = torch.arange((plan.hidden_size + 1) // 2, dtype=torch.float64)
+            self.turns = (float(plan.sinusoid_base) ** (-2.0 * i / plan.hidden_size) / (2.0 * math.pi)).to(self.device)
         self._embedding_joins_again = any(entry.add_embedding for entry in plan.schedule)
         for block in self.blocks:
             block.bind(weights)
@@ -226,7 +231,7 @@ class Model:
         # the norm that reads the stream first at every stop (and the final norm after the last)
         first_norms = [getattr(self.blocks[entry.layer], "mixer_norm", None) for entry in plan.schedule] + [self.final_norm]
         entry_fold = getattr(self.blocks[plan.schedule[0].layer], "entry_fold", None) if plan.schedule and T else None
-        own_kernel = plan.pair_embedding is not None or self.position_table is not None
+        own_kernel = plan.pair_embedding is not None or self.position_table is not None or self.turns is not None
         fold = entry_fold(T) if entry_fold is not None and not own_kernel else None
         if self.position_table is not None:
             if plan.pair_embedding is not None or copies > 1:
@@ -234,6 +239,10 @@ class Model:
             if ctx.q_lens and max(p + n for p, n in zip(ctx.past_lens, ctx.q_lens)) > plan.max_positions:
                 raise ValueError(f"a sequence passes the {plan.max_positions} positions the model has rows for")
             K.embedding_positions(residual, self.embedding, token_ids, self.position_table, ctx.positions, plan.embedding_scale)
+        elif self.turns is not None:
+            K.embedding_sinusoids(residual, self.embedding, token_ids, self.turns, ctx.positions, plan.embedding_scale)
+            if copies > 1:
+                K.hyper_spread(stream.residual, residual, copies)
         elif fold is not None:
             # the first block's norm lets the embedding prepare its rows (see parts.OwedRows)
             norm, weight, eps = fold

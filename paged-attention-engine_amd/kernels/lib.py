@@ -72,7 +72,7 @@ def _declare(lib) -> None:
         "pae_gemm_skinny_gated": [P, L, P, L, P, I, I, I, I, P, P, I, P],
         "pae_paged_attention_generic": [I, P, L, P, L, P, P, P, P, P, I, I, I, I, I, I, F, I, P],
         "pae_paged_attention_capped": [I, P, L, P, L, P, P, P, P, P, I, I, I, I, I, I, I, F, I, F, P, P],
-        "pae_qk_norm_rotate_store": [I, P, L, I, I, I, I, I, P, P, I, F, I, I, P, F, P, P, P, I, I, P, P, I, I, P],
+        "pae_qk_norm_rotate_store": [I, P, L, I, I, I, I, I, P, P, I, F, I, I, P, F, P, P, P, I, I, P, P, I, I, F, I, P, L, F, P],
         "pae_paged_attention_masked": [I, P, L, P, L, P, P, P, P, P, I, I, I, I, I, I, I, F, I, F, P, I, P, P, L, I, I, P],
         "pae_hyper_norm": [I, P, I, P, I, L, P, I, P, P, P, P, I, F, P, P, I, I, I, P],
         "pae_hyper_spread": [P, P, I, I, I, P],
@@ -93,14 +93,14 @@ def _declare(lib) -> None:
         "pae_gemm_plain_batched": [I, I, P, L, L, P, L, L, P, L, P, I, I, I, I, I, P],
         "pae_rows_from_residual": [I, P, P, L, P],
         "pae_norm_scale_add": [I, P, P, I, L, P, I, F, F, P, I, I, P],
-        "pae_activation": [I, P, L, I, P],
+        "pae_activation": [I, P, L, I, P, I, I, P],
         "pae_delta_rule_step": [I, P, L, I, I, P, P, P, P, P, P, L, I, I, I, I, I, P, P, F, P, L, P, I, F, P, P,
                                 P, L, I, P, L, P, L, I, P],
         "pae_matrix_memory_step": [I, P, L, P, L, P, I, I, P, P, I, I, I, F, P, L, P, L, P, I, F, F, P, P, P],
         "pae_embedding_pairs": [I, P, P, P, P, P, P, P, P, I, I, I, F, I, I, I, P],
         "pae_sum_norm2": [I, P, I, P, P, P, P, P, P, I, P, I, F, P, P, P, I, I, I, P],
         "pae_project_f32": [I, P, L, P, L, P, P, I, I, I, I, P],
-        "pae_moe_route": [P, I, I, I, I, I, F, P, P, P, P],
+        "pae_moe_route": [P, I, I, I, I, I, F, P, L, I, I, P, P, P],
         "pae_norm_join": [I, P, I, P, P, P, P, P, P, I, F, P, I, F, P, P, I, I, P],
         "pae_linear_attention_step": [I, P, L, P, L, P, I, F, P, L, I, I, I, P, P, I, I, I, P, L, P, I, F, P, P, P],
         "pae_fixed_decay_chunk": [I],
@@ -110,6 +110,7 @@ def _declare(lib) -> None:
         "pae_norm_join_conv_supported": [I],
         "pae_norm_join_conv": [I, P, P, I, L, P, I, F, F, P, P, L, P, P, I, P, I, I, P],
         "pae_embedding_positions": [I, P, P, P, P, P, I, I, I, F, P],
+        "pae_embedding_sinusoids": [I, P, P, P, P, P, I, I, I, F, P],
         "pae_token_gate": [I, P, P, L, P, P, I, I, I, P],
         "pae_moe_gate_up": [I, P, P, L, P, P, P, I, I, I, I, I, P],
         "pae_moe_down": [I, P, P, P, P, P, I, I, I, I, P],
@@ -126,8 +127,8 @@ def _declare(lib) -> None:
         "pae_attn_decode_split": [],
         "pae_attn_decode_biased_bf16": [P, L, P, L, P, P, P, I, P, I, I, I, I, I, F, I, I, P, P, L, P, P, P],
         "pae_attn_prefill_biased_bf16": [P, L, P, L, P, P, P, I, P, P, I, I, I, I, I, F, I, I, P, P, L, P],
-        "pae_attn_decode_capped_bf16": [P, L, P, L, P, P, P, I, P, I, I, I, I, I, F, I, F, P, P, P, P],
-        "pae_attn_prefill_capped_bf16": [P, L, P, L, P, P, P, I, P, P, I, I, I, I, I, F, I, F, P, P],
+        "pae_attn_decode_capped_bf16": [P, L, P, L, P, P, P, I, P, I, I, I, I, I, F, I, F, P, P, L, P, P, P],
+        "pae_attn_prefill_capped_bf16": [P, L, P, L, P, P, P, I, P, P, I, I, I, I, I, F, I, F, P, P, L, P],
         "pae_attn_prefill_bf16": [P, L, P, L, P, P, P, I, P, P, I, I, I, I, I, F, I, P],
         "pae_program_phase_bytes": [],
         "pae_program_barrier_bytes": [],
@@ -230,6 +231,22 @@ def embedding_positions(out: torch.Tensor, table: torch.Tensor, ids: torch.Tenso
         assert t.dtype == torch.int32 and t.numel() == T and t.is_contiguous()
     _check(library().pae_embedding_positions(code_of(table.dtype), out.data_ptr(), table.data_ptr(), ids.data_ptr(),
                                              rows.data_ptr(), positions.data_ptr(), T, H, table.shape[0], float(scale),
+                                             _stream()))
+
+
+def embedding_sinusoids(out: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, turns: torch.Tensor,
+                        positions: torch.Tensor, scale: float = 1.0) -> None:
+    """out[t] = scale * table[ids[t]] + P(positions[t]) as float32, with P(p)[2i] = sin(2 pi p turns[i]) and
+    P(p)[2i + 1] = cos of the same; `turns` float64 [ceil(H / 2)]: the frequencies in turns a position."""
+    _not_while_recording("embedding_sinusoids")
+    _gpu(out, table, ids, turns, positions)
+    T, H = out.shape
+    assert out.dtype == torch.float32 and out.is_contiguous() and table.is_contiguous() and table.shape[1] == H
+    assert turns.dtype == torch.float64 and turns.numel() == (H + 1) // 2 and turns.is_contiguous()
+    for t in (ids, positions):
+        assert t.dtype == torch.int32 and t.numel() == T and t.is_contiguous()
+    _check(library().pae_embedding_sinusoids(code_of(table.dtype), out.data_ptr(), table.data_ptr(), ids.data_ptr(),
+                                             turns.data_ptr(), positions.data_ptr(), T, H, table.shape[0], float(scale),
                                              _stream()))
 
 
@@ -1375,13 +1392,16 @@ def qk_norm_rotate_store(qkv: torch.Tensor, nh: int, nkv: int, hd: int, vd: int,
                          k_weight: Optional[torch.Tensor], eps: float, rot: int, interleaved: bool,
                          cos_sin: Optional[torch.Tensor], magnitude: float, positions: torch.Tensor,
                          tok_seq: Optional[torch.Tensor], block_tables: Optional[torch.Tensor], block_size: int,
-                         k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], per_head: bool = False) -> None:
+                         k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], per_head: bool = False,
+                         temperature=None, mix=None) -> None:
     """Rows [q: nh x hd | k: nkv x hd | v: nkv x vd]: with weights, q and k are each divided by the root
     mean square of their whole projection and multiplied by the weight (`per_head`: every head by its own root
     mean square, and the weights are hd numbers that the heads share); the first `rot` features of
     every q and k head are rotated by `cos_sin` times `magnitude` (pairs (2i, 2i+1) if `interleaved`,
     else (i, i + rot/2)); queries are written back in place, keys and values to their cache slots
-    (`k_cache` None: nkv must be 0 and nothing is stored)."""
+    (`k_cache` None: nkv must be 0 and nothing is stored).  `temperature` = (coef, every): queries are multiplied
+    by 1 + coef ln(floor((p + 1) / every) + 1) at position p.  `mix` = (first [T, nkv * vd], share): the values stored
+    are (1 - share) v + share first, `first` a view of rows in qkv's type."""
     _not_while_recording("qk_norm_rotate_store")
     _gpu(qkv, q_weight, k_weight, cos_sin, positions, tok_seq, block_tables, k_cache, v_cache)
     T = qkv.shape[0]
@@ -1395,6 +1415,12 @@ def qk_norm_rotate_store(qkv: torch.Tensor, nh: int, nkv: int, hd: int, vd: int,
         assert nkv == 0 or (k_weight is not None and k_weight.numel() == (hd if per_head else nkv * hd)
                             and k_weight.dtype == q_weight.dtype and k_weight.is_contiguous())
         wf = _param(q_weight)[1]
+    coef, every = (0.0, 0) if temperature is None else temperature
+    assert temperature is None or every > 0
+    first, share = (None, 0.0) if mix is None else mix
+    if first is not None:
+        _gpu(first)
+        assert write and first.shape == (T, nkv * vd) and first.stride(1) == 1 and first.dtype == qkv.dtype
     max_blocks = 0
     if write:
         assert k_cache.dtype == qkv.dtype == v_cache.dtype
@@ -1406,7 +1432,8 @@ def qk_norm_rotate_store(qkv: torch.Tensor, nh: int, nkv: int, hd: int, vd: int,
         code_of(qkv.dtype), qkv.data_ptr(), qkv.stride(0), T, nh, nkv, hd, vd, _ptr(q_weight), _ptr(k_weight), wf,
         float(eps), rot, 1 if interleaved else 0, _ptr(cos_sin) if rot else None, float(magnitude),
         positions.data_ptr(), _ptr(tok_seq), _ptr(block_tables), max_blocks, block_size, _ptr(k_cache), _ptr(v_cache),
-        1 if write else 0, 1 if (per_head and q_weight is not None) else 0, _stream()))
+        1 if write else 0, 1 if (per_head and q_weight is not None) else 0, float(coef), int(every), _ptr(first),
+        first.stride(0) if first is not None else 0, float(share), _stream()))
 
 
 def rows_from_residual(residual: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
@@ -1447,15 +1474,19 @@ def norm_scale_add(residual: torch.Tensor, y: torch.Tensor, weight: torch.Tensor
                                         float(eps), float(scale), _ptr(next_rows), T, H, _stream()))
 
 
-ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2}
+ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu2": 3}
 
 
-def activation(x: torch.Tensor, kind: str) -> None:
-    """x <- act(x) in place, computed in float32: "gelu" (by erf), "gelu_tanh", "silu"."""
+def activation(x: torch.Tensor, kind: str, bias: Optional[torch.Tensor] = None) -> None:
+    """x <- act(x + bias) in place, computed in float32: "gelu" (by erf), "gelu_tanh", "silu", "relu2" (the square of
+    relu); `bias`: one number per column of the rows x, or none."""
     _not_while_recording("activation")
-    _gpu(x)
+    _gpu(x, bias)
     assert x.is_contiguous() and kind in ACTIVATIONS
-    _check(library().pae_activation(code_of(x.dtype), x.data_ptr(), x.numel(), ACTIVATIONS[kind], _stream()))
+    assert bias is None or (bias.numel() == x.shape[-1] and bias.is_contiguous())
+    bp, bf = _param(bias)
+    _check(library().pae_activation(code_of(x.dtype), x.data_ptr(), x.numel(), ACTIVATIONS[kind], bp, bf, x.shape[-1],
+                                    _stream()))
 
 
 def delta_rule_step(proj: torch.Tensor, out: torch.Tensor, tok_seq: torch.Tensor, positions: torch.Tensor,
@@ -1810,21 +1841,27 @@ def project_f32(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] =
 
 
 def moe_route(logits: torch.Tensor, groups: int, keep: int, top: int, scale: float,
-              choice_bias: Optional[torch.Tensor] = None):
+              choice_bias: Optional[torch.Tensor] = None, among_chosen: bool = False, shared_pieces: int = 0):
     """(chosen int32 [T, top], weights float32 [T, top]) from router logits float32 [T, E]: scores are the softmax
     over all experts; only experts of the `keep` best of `groups` equal groups of neighbours (a group's score is
     its largest) can be chosen; the weights are the chosen scores times `scale`.  With `choice_bias` (float32 [E])
-    experts and groups are compared by score + bias; the weights stay the scores."""
+    experts and groups are compared by score + bias; the weights stay the scores.  With `among_chosen` experts are
+    compared by their logits and weighted by the softmax over the chosen logits alone, times `scale` (one group, no bias).
+    With `shared_pieces` P the logits have one column more, z; every token then also gets the experts E .. E + P - 1
+    (pieces of an expert that all tokens use), each weighted by sigmoid(z): the results are [T, top + P]."""
     _not_while_recording("moe_route")
     _gpu(logits, choice_bias)
     T, E = logits.shape
+    E -= 1 if shared_pieces else 0
     assert logits.dtype == torch.float32 and logits.is_contiguous()
+    assert not among_chosen or (groups == 1 and choice_bias is None)
     if choice_bias is not None:
         assert choice_bias.dtype == torch.float32 and choice_bias.numel() == E and choice_bias.is_contiguous()
-    chosen = torch.empty((T, top), dtype=torch.int32, device=logits.device)
-    weights = torch.empty((T, top), dtype=torch.float32, device=logits.device)
+    chosen = torch.empty((T, top + shared_pieces), dtype=torch.int32, device=logits.device)
+    weights = torch.empty((T, top + shared_pieces), dtype=torch.float32, device=logits.device)
     _check(library().pae_moe_route(logits.data_ptr(), T, E, int(groups), int(keep), int(top), float(scale),
-                                   _ptr(choice_bias), chosen.data_ptr(), weights.data_ptr(), _stream()))
+                                   _ptr(choice_bias), logits.stride(0), 1 if among_chosen else 0, int(shared_pieces),
+                                   chosen.data_ptr(), weights.data_ptr(), _stream()))
     return chosen, weights
 
 
@@ -1882,14 +1919,18 @@ def mfma_attention_supported(dtype: torch.dtype, nh: int, nkv: int, hd: int, bs:
 def attn_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                 dec_work: torch.Tensor, block_tables: torch.Tensor, nh: int, nkv: int, hd: int, scale: float,
                 window: int, softcap: float = 0.0, sinks: Optional[torch.Tensor] = None, chunked: bool = False,
-                slopes: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> None:
+                slopes: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
+                head_gate: Optional[torch.Tensor] = None) -> None:
     """Attention of the single new token of each sequence listed in `dec_work` over that sequence's
     cached keys: split over the keys, then merged.  dec_work[i] = (flat row of the token, its
     position, row of its sequence in `block_tables`, 0).  `softcap` > 0 caps the scores
     (s <- softcap tanh(s / softcap)); `sinks` (float32 [nh]) join each head's softmax denominator.
-    `chunked`, `slopes`, `gate`: as in `paged_attention_masked` (not together with a cap or sinks)."""
-    _gpu(out, q, k_cache, v_cache, dec_work, block_tables, sinks, slopes, gate)
-    wide = bool(softcap) or sinks is not None
+    `chunked`, `slopes`, `gate`: as in `paged_attention_masked` (not together with a cap, sinks or a head gate);
+    `head_gate` [T, >= nh] bfloat16 rows: a head's output is multiplied by its number's sigmoid."""
+    _gpu(out, q, k_cache, v_cache, dec_work, block_tables, sinks, slopes, gate, head_gate)
+    if head_gate is not None:
+        _check_head_gate(head_gate, q, nh)
+    wide = bool(softcap) or sinks is not None or head_gate is not None
     biased = chunked or slopes is not None or gate is not None
     assert not (wide and biased)
     if sinks is not None:
@@ -1916,11 +1957,12 @@ def attn_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cac
             int(window), 1 if chunked else 0, _ptr(slopes), gp, gs, part_acc.data_ptr(), part_ml.data_ptr(), _stream()))
         return
     if wide:
-        _not_while_recording("attn_decode with a score cap or sinks")
+        _not_while_recording("attn_decode with a score cap, sinks or a head gate")
         _check(library().pae_attn_decode_capped_bf16(
             out.data_ptr(), out.stride(0), q.data_ptr(), q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
             dec_work.data_ptr(), n, block_tables.data_ptr(), block_tables.shape[1], bs, nh, nkv, hd, float(scale),
-            int(window), float(softcap), _ptr(sinks), part_acc.data_ptr(), part_ml.data_ptr(), _stream()))
+            int(window), float(softcap), _ptr(sinks), _ptr(head_gate), head_gate.stride(0) if head_gate is not None else 0,
+            part_acc.data_ptr(), part_ml.data_ptr(), _stream()))
         return
     if _RECORDING is not None:
         _RECORDING.room(2)  # the splits' partial results, then their merge
@@ -1944,15 +1986,17 @@ def attn_prefill(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_ca
                  tiles: torch.Tensor, positions: torch.Tensor, block_tables: torch.Tensor,
                  nh: int, nkv: int, hd: int, scale: float, window: int, softcap: float = 0.0,
                  sinks: Optional[torch.Tensor] = None, chunked: bool = False, slopes: Optional[torch.Tensor] = None,
-                 gate: Optional[torch.Tensor] = None) -> None:
+                 gate: Optional[torch.Tensor] = None, head_gate: Optional[torch.Tensor] = None) -> None:
     """Attention of runs of consecutive tokens; tiles[t] = (table row of the sequence, first
     flat token, number of tokens <= PREFILL_TILE).  One workgroup per run and head, whose
     wavefronts share out the keys; workgroups start in the order of `tiles`, so the runs with
-    the most keys should come first.  `softcap`, `sinks`, `chunked`, `slopes` and `gate` as in `attn_decode`."""
+    the most keys should come first.  `softcap`, `sinks`, `chunked`, `slopes`, `gate` and `head_gate` as in `attn_decode`."""
     _not_while_recording("attn_prefill")
-    _gpu(out, q, k_cache, v_cache, tiles, positions, block_tables, sinks, slopes, gate)
+    _gpu(out, q, k_cache, v_cache, tiles, positions, block_tables, sinks, slopes, gate, head_gate)
+    if head_gate is not None:
+        _check_head_gate(head_gate, q, nh)
     biased = chunked or slopes is not None or gate is not None
-    assert not (biased and (softcap or sinks is not None))
+    assert not (biased and (softcap or sinks is not None or head_gate is not None))
     if sinks is not None:
         assert sinks.dtype == torch.float32 and sinks.numel() == nh and sinks.is_contiguous()
     bs = k_cache.shape[2]
@@ -1972,7 +2016,8 @@ def attn_prefill(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_ca
     _check(library().pae_attn_prefill_capped_bf16(
         out.data_ptr(), out.stride(0), q.data_ptr(), q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
         tiles.data_ptr(), tiles.shape[0], positions.data_ptr(), block_tables.data_ptr(), block_tables.shape[1],
-        bs, nh, nkv, hd, float(scale), int(window), float(softcap), _ptr(sinks), _stream()))
+        bs, nh, nkv, hd, float(scale), int(window), float(softcap), _ptr(sinks), _ptr(head_gate),
+        head_gate.stride(0) if head_gate is not None else 0, _stream()))
 
 
 def sample(tokens: torch.Tensor, logits: torch.Tensor, temperature: Optional[torch.Tensor],

@@ -24,9 +24,13 @@ softcap * tanh(score / softcap), and a learned sink per query head that joins th
 denominator as exp(sink) without a key or a value (`sinks`), or one number that is every head's sink
 (`fixed_sink`: with 0 the denominator is one larger than the sum of exponentials), or an RMS norm of
 every query and key head by itself with one weight that the heads share (`qk_norm = "per_head"`).
-A spec with any of them takes the
-path `_forward_wide`: the projection, then one kernel that norms, rotates and stores, then the
-attention kernel that knows caps, sinks and value widths.
+Also a temperature on the queries that
+grows with the position (`temperature`), values mixed with those of an earlier layer (`value_mix`: the layer
+called "source" leaves its values for the step where the layers called "mixed" find them, and the mixed values are
+what is cached), and a gate of one number per head, sigmoid(W_g x)_h on head h's output before W_o (`head_gate_name`:
+its rows ride in the one product).  A spec with any of them takes the
+path `_forward_wide`: the projection, then one kernel that norms, rotates, mixes and stores, then the
+attention kernel that knows caps, sinks, gates and value widths.
 
 And for designs that have them (`MixerSpec.convolved`, the path `_forward_convolved`): a short causal
 convolution over time on every channel of q, k and v right after the projection, whose last
@@ -50,6 +54,7 @@ from .delta import sequence_runs
 from .linear import Linear, rows_a_graph_may_hold
 
 WORK_LISTS = ("paged attention work lists", K.PREFILL_TILE)
+SOURCE_VALUES = "values of the layer that others mix in"  # the key of a step's memo under which they wait
 CONV_LISTS = ("paged attention work lists and sequence runs", K.PREFILL_TILE)
 
 
@@ -72,7 +77,7 @@ def attention_work_lists(shape: StepShape):
 
 
 def attend_paged(attn, q, k_cache, v_cache, positions, tok_seq, table, work, num_heads: int, num_kv_heads: int,
-                 head_dim: int, value_dim: int, scale: float, window: int, softcap: float, sinks) -> None:
+                 head_dim: int, value_dim: int, scale: float, window: int, softcap: float, sinks, head_gate=None) -> None:
     """Attention of a step's queries over the paged cache into `attn`: with `work` (the device lists of
     `attention_work_lists`) on the matrix cores, single tokens by the decode kernel and runs of tokens by
     the prefill kernel; without, by the kernel that takes any shape and precision."""
@@ -80,9 +85,12 @@ def attend_paged(attn, q, k_cache, v_cache, positions, tok_seq, table, work, num
         geometry = (num_heads, num_kv_heads, head_dim, scale, window, softcap, sinks)
         decode_work, prefill_tiles = work["decode_work"], work["prefill_tiles"]
         if decode_work.numel():
-            K.attn_decode(attn, q, k_cache, v_cache, decode_work, table, *geometry)
+            K.attn_decode(attn, q, k_cache, v_cache, decode_work, table, *geometry, head_gate=head_gate)
         if prefill_tiles.numel():
-            K.attn_prefill(attn, q, k_cache, v_cache, prefill_tiles, positions, table, *geometry)
+            K.attn_prefill(attn, q, k_cache, v_cache, prefill_tiles, positions, table, *geometry, head_gate=head_gate)
+    elif head_gate is not None:
+        K.paged_attention_masked(attn, q, k_cache, v_cache, positions, tok_seq, table, num_heads, num_kv_heads,
+                                 head_dim, value_dim, scale, window, softcap=softcap, sinks=sinks, head_gate=head_gate)
     else:
         K.paged_attention_capped(attn, q, k_cache, v_cache, positions, tok_seq, table, num_heads, num_kv_heads,
                                  head_dim, value_dim, scale, window, softcap, sinks)
@@ -104,7 +112,14 @@ class PagedAttention(Part):
             raise ValueError("an attention has learned sinks or one fixed sink, not both")
         if spec.mask not in ("window", "chunk"):
             raise ValueError(f"mask '{spec.mask}' is not known (known: window, chunk)")
+        if spec.value_mix not in (None, "source", "mixed"):
+            raise ValueError(f"value_mix '{spec.value_mix}' is not known (known: source, mixed)")
+        if spec.temperature is not None and spec.temperature.every <= 0:
+            raise ValueError(f"a query temperature that grows every {spec.temperature.every} positions")
         if spec.convolved:
+            if spec.temperature is not None or spec.value_mix is not None or spec.head_gate_name is not None:
+                raise ValueError("an attention with convolutions, chunks, distance bias or a gate per feature takes no "
+                                 "query temperature, value mixing or gate per head")
             if (spec.position is not None or spec.qk_norm in ("projection", "per_head") or spec.sinks or spec.softcap
                     or spec.fixed_sink is not None):
                 raise ValueError("an attention with convolutions, per-head norms, chunks, distance bias or a gate "
@@ -210,6 +225,10 @@ class PagedAttention(Part):
             out[prefix + s.k_norm_name] = ScaleShape((s.num_kv_heads * s.head_dim,))
         if s.sinks:
             out[prefix + s.sink_name] = (s.num_heads,)
+        if s.value_mix == "mixed":
+            out[prefix + s.value_mix_name] = ()
+        if s.head_gate_name is not None:
+            out[prefix + s.head_gate_name + s.weight_suffix] = (s.num_heads, s.hidden_size)
         if s.qkv_bias:
             out[prefix + s.q_name + s.bias_suffix] = (s.num_heads * s.head_dim,)
             out[prefix + s.k_name + s.bias_suffix] = (s.num_kv_heads * s.head_dim,)
@@ -245,9 +264,19 @@ class PagedAttention(Part):
         if s.convolved:
             return self._bind_convolved(prefix, weights)
         names = (s.q_name, s.k_name, s.v_name)
-        w = torch.cat([weights[prefix + n + s.weight_suffix] for n in names], dim=0)
+        rows = [weights[prefix + n + s.weight_suffix] for n in names]
+        if s.head_gate_name is not None:
+            # the gate reads the same input: its rows ride in the same product, without a bias; zero rows behind them
+            # keep the product's own rows on 16-byte boundaries
+            gate = weights[prefix + s.head_gate_name + s.weight_suffix]
+            width = sum(r.shape[0] for r in rows) + s.num_heads
+            rows += [gate, torch.zeros((-width % 8, s.hidden_size), dtype=gate.dtype, device=gate.device)]
+        w = torch.cat(rows, dim=0)
         b = (torch.cat([weights[prefix + n + s.bias_suffix] for n in names], dim=0) if s.qkv_bias else None)
+        if b is not None and b.shape[0] < w.shape[0]:
+            b = torch.cat([b, torch.zeros(w.shape[0] - b.shape[0], dtype=b.dtype, device=b.device)])
         self.qkv = Linear(self.matrix(w), None if b is None else self.vector(b))
+        self.value_share = float(weights[prefix + s.value_mix_name]) if s.value_mix == "mixed" else 0.0
         nq = s.num_heads * s.head_dim
         self.q_only = Linear(self.qkv.weight[:nq], None if b is None else self.qkv.bias[:nq])
         ob = weights[prefix + s.o_name + s.bias_suffix] if s.out_bias else None
@@ -308,21 +337,36 @@ class PagedAttention(Part):
         table = ctx.block_tables[ctx.cache.group_of(ctx.cache_entry)]
         if ctx.writes_cache:
             qkv, nkv, k_cache, v_cache = self.qkv(x), s.num_kv_heads, pages["k"], pages["v"]
+        elif s.value_mix is not None or s.head_gate_name is not None:
+            raise ValueError("an attention with value mixing or a gate per head reads its own pages, not another stop's")
         else:
             qkv, nkv, k_cache, v_cache = self.q_only(x), 0, None, None
         rotary = getattr(self.position, "rotary_table", None)
         if rotary is None and s.position is not None:
             raise ValueError("an attention with value widths, caps, sinks or query/key norms rotates by a table")
         rot, cos_sin = rotary(ctx) if rotary is not None else (0, None)
+        first_value = s.num_heads * s.head_dim + nkv * s.head_dim
+        values = qkv[:, first_value:first_value + nkv * s.v_dim]
+        mix = None
+        if s.value_mix == "source":  # (the row keeps the layer's own values, whatever is cached)
+            ctx.memo[SOURCE_VALUES] = values
+        elif s.value_mix == "mixed":
+            if SOURCE_VALUES not in ctx.memo:
+                raise ValueError("a layer mixes in the values of an earlier one, but no earlier one left any")
+            mix = (ctx.memo[SOURCE_VALUES], self.value_share)
         K.qk_norm_rotate_store(qkv, s.num_heads, nkv, s.head_dim, s.v_dim, self.q_norm, self.k_norm if nkv else None,
                                s.qk_norm_eps, rot, bool(getattr(self.position, "interleaved", False)), cos_sin,
                                float(getattr(self.position, "magnitude", 1.0)), ctx.positions,
                                ctx.tok_seq if nkv else None, table if nkv else None, ctx.cache.block_size,
-                               k_cache, v_cache, per_head=s.qk_norm == "per_head")
+                               k_cache, v_cache, per_head=s.qk_norm == "per_head",
+                               temperature=None if s.temperature is None else (s.temperature.coef, s.temperature.every), mix=mix)
+        gate = None
+        if s.head_gate_name is not None:
+            gate = qkv[:, first_value + nkv * s.v_dim:first_value + nkv * s.v_dim + s.num_heads]
         attn = torch.empty((qkv.shape[0], s.num_heads * s.v_dim), dtype=qkv.dtype, device=qkv.device)
         work = ctx.memo.get(WORK_LISTS) if self._matrix_cores(ctx.cache.block_size) else None
         attend_paged(attn, qkv, pages["k"], pages["v"], ctx.positions, ctx.tok_seq, table, work, s.num_heads,
-                     s.num_kv_heads, s.head_dim, s.v_dim, s.scale, s.window or 0, s.softcap or 0.0, self.sinks)
+                     s.num_kv_heads, s.head_dim, s.v_dim, s.scale, s.window or 0, s.softcap or 0.0, self.sinks, gate)
         return self.out.branch(attn, ctx.sink)
 
     def _forward_convolved(self, ctx, x):

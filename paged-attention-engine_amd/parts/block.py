@@ -400,9 +400,9 @@ class SandwichBlock:
             self.feed_forward = build_part(FEED_FORWARDS, "feed-forward", layer_spec.feed_forward, dtype, device)
             self.feed_forward_out_norm = build_part(NORMS, "norm", layer_spec.feed_forward_out_norm, dtype, device)
         for norm in (self.mixer_norm, self.mixer_out_norm, self.feed_forward_norm, self.feed_forward_out_norm):
-            if norm is not None and (not isinstance(norm, RMSNorm) or norm.spec.weight_offset):
+            if norm is not None and not isinstance(norm, RMSNorm):
                 raise ValueError(f"the norm '{norm.spec.kind}' cannot ride in the kernel that joins a sublayer's output "
-                                 "(an RMS norm with a plain weight can)")
+                                 "(an RMS norm can)")
         self.side = None
         if layer_spec.token_side is not None:
             self.side = TokenSide(layer_spec.token_side, dtype, device, layer_spec.mixer_norm.size)
@@ -456,11 +456,9 @@ class SandwichBlock:
 
     def _next_first_norm(self, stream: ResidualStream):
         """The first norm of the block that follows, if that block takes its rows prepared (the model says so) and
-        the norm is one the joining kernel can form (an RMS norm with a plain weight); else None."""
+        the norm is one the joining kernel can form (an RMS norm); else None."""
         norm = stream.next_norm if stream.prepared_wanted_next else None
-        if norm is None or not isinstance(norm, type(self.mixer_norm)) or norm.spec.weight_offset:
-            return None
-        return norm
+        return norm if isinstance(norm, type(self.mixer_norm)) else None
 
     def forward(self, ctx, stream: ResidualStream) -> None:
         if stream.pending is not None or stream.owed is not None or stream.copies != 1:

@@ -81,7 +81,8 @@ class Linear:
         return self._library(x, with_bias=False)
 
     def branch(self, x: torch.Tensor, sink=None) -> Optional[torch.Tensor]:
-        """The product as a residual branch's output: [M, N] in x's dtype, or float32
+        """The product as a residual branch's output: [M, N] in x's dtype (few rows with a bias: k ranges
+        that are added up inside the kernel, see `whole_sum_splits`), or float32
         partial sums [P, M, N] that the next norm adds up in order (no bias then).  With a `sink`
         whose norm can be folded, the few-row product adds itself into the residual instead and
         prepares the following product's rows; nothing is returned then."""
@@ -101,6 +102,11 @@ class Linear:
                 return None
             out = torch.empty((splits, x.shape[0], self.out_features), dtype=torch.float32, device=x.device)
             K.gemm_skinny(out, x, self.weight, None, K.EPI_F32, splits)
+            return out
+        if x.dtype == torch.bfloat16 and x.shape[0] and K.skinny_supported(x, self.weight):
+            out = torch.empty((x.shape[0], self.out_features), dtype=x.dtype, device=x.device)
+            K.gemm_skinny(out, x, self.weight, self.bias, K.EPI_BF16,
+                          K.whole_sum_splits(self.out_features, self.in_features, x.shape[0]))
             return out
         return self(x)
 

@@ -2,7 +2,7 @@
 (engine/model.py:317-320 of the reference) or another of `kernels.lib.ACTIVATIONS` by the spec's
 `activation`.  gate and up are one product over
 concatenated weights; the gate is applied in float32 and rounded once.  "dense", the plain
-one: down(act(up(x))), act one of `kernels.lib.ACTIVATIONS`, applied in float32."""
+one: down(act(up(x))), with or without biases, act one of `kernels.lib.ACTIVATIONS`, applied in float32."""
 
 from __future__ import annotations
 
@@ -79,8 +79,8 @@ class SwiGLU(Part):
 
 @register_feed_forward("dense")
 class DenseFeedForward(Part):
-    """down(act(up(x))), no gate, no biases.  `spec.activation`: "gelu" (the exact one, by erf),
-    "gelu_tanh" or "silu"."""
+    """down(act(up(x))), no gate; both products add a bias if the spec says so.  `spec.activation`: "gelu" (the
+    exact one, by erf), "gelu_tanh", "silu" or "relu2" (the square of relu)."""
 
     graph_safe = True
 
@@ -95,23 +95,31 @@ class DenseFeedForward(Part):
 
     def tensors(self, prefix):
         s = self.spec
-        return {prefix + s.up_name + s.weight_suffix: (s.intermediate_size, s.hidden_size),
-                prefix + s.down_name + s.weight_suffix: (s.hidden_size, s.intermediate_size)}
+        out = {prefix + s.up_name + s.weight_suffix: (s.intermediate_size, s.hidden_size),
+               prefix + s.down_name + s.weight_suffix: (s.hidden_size, s.intermediate_size)}
+        if s.bias:
+            out[prefix + s.up_name + s.bias_suffix] = (s.intermediate_size,)
+            out[prefix + s.down_name + s.bias_suffix] = (s.hidden_size,)
+        return out
 
     def bind(self, prefix, weights):
         s = self.spec
-        self.up = Linear(self.matrix(weights[prefix + s.up_name + s.weight_suffix]))
-        self.down = Linear(self.matrix(weights[prefix + s.down_name + s.weight_suffix]))
+        bias = lambda name: self.vector(weights[prefix + name + s.bias_suffix]) if s.bias else None
+        self.up = Linear(self.matrix(weights[prefix + s.up_name + s.weight_suffix]), bias(s.up_name))
+        self.down = Linear(self.matrix(weights[prefix + s.down_name + s.weight_suffix]), bias(s.down_name))
 
     def forward(self, ctx, x):
         """Up to 64 rows the activation runs in the up product's epilogue, on its float32 sums; above,
-        the platform library's product is followed by the activation kernel."""
+        the platform library's product is followed by the activation kernel, which adds the bias first."""
         x = plain_rows(x)
         if x.shape[0] and K.skinny_supported(x, self.up.weight):
             act = torch.empty((x.shape[0], self.spec.intermediate_size), dtype=x.dtype, device=x.device)
             splits = K.whole_sum_splits(self.spec.intermediate_size, self.spec.hidden_size, x.shape[0])
-            K.gemm_skinny_act(act, x, self.up.weight, self.spec.activation, splits)
+            K.gemm_skinny_act(act, x, self.up.weight, self.spec.activation, splits, self.up.bias)
         else:
-            act = self.up(x)
-            K.activation(act, self.spec.activation)
+            act = self.up.without_bias(x)
+            bias = self.up.bias if act is not None else None
+            if act is None:
+                act = self.up(x)
+            K.activation(act, self.spec.activation, bias)
         return self.down.branch(act, getattr(ctx, "sink", None))

@@ -54,7 +54,7 @@ class RMSNorm(Part):
         and prepared this norm's rows, they are returned as they are (`OwedRows`): no kernel runs."""
         if stream.copies > 1 or stream.join is not None:
             return self.forward_copies(stream, stream.sum_weights, rows)
-        if isinstance(stream.pending, BranchTerms):
+        if isinstance(stream.pending, BranchTerms) or (self.spec.weight_offset and stream.owed is None):  # (rounds once)
             return self.forward_pair(stream, None, rows)[0]
         if stream.owed is not None:
             owed, mine = stream.owed, stream.owed_to is self

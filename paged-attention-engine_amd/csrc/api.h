@@ -137,11 +137,14 @@ int pae_delta_rule_step(int dtype, const void* proj, int64_t row_stride, int num
 int64_t pae_delta_rule_work_floats(int num_tokens, int G, int H, int D, int V, int channel_decay);
 // a matrix memory with exponential gates over a step's projected rows: see matrix_memory.hip
 int pae_matrix_memory_step(int dtype, const void* proj, int64_t row_stride, const void* gate_in, int64_t gate_stride,
-                           const float* gate_logits, int num_tokens, int num_seqs, const int* seq_runs, const int* slots,
-                           int H, int D, int V, float gate_cap, float* state, int64_t state_slot_stride, float* maximum,
-                           int64_t max_slot_stride, const void* norm_w, int w_is_f32, float norm_eps, float floor_eps,
-                           float* work, void* out, hipStream_t stream);
-int64_t pae_matrix_memory_work_floats(int num_tokens, int H, int D, int V);
+                           const float* gate_logits, const void* x, int64_t ldx, const void* gate_w, const float* gate_b,
+                           int hidden, int num_tokens, const int* serial, int num_serial, const int* chunks, int num_chunks,
+                           const int* scans, int num_scans, const int* slots, int H, int D, int V, float gate_cap,
+                           float* state, int64_t state_slot_stride, float* maximum, int64_t max_slot_stride,
+                           const void* norm_w, int w_is_f32, float norm_eps, float floor_eps, float* work, void* out,
+                           hipStream_t stream);
+int64_t pae_matrix_memory_work_floats(int num_tokens, int num_chunks, int H, int D, int V);
+int pae_matrix_memory_chunk(int D);
 // the embedding with a hashed table of token pairs added: see hashed_embedding.hip
 int pae_embedding_pairs(int dtype, float* out, const void* table, const void* pair_table, const int* ids,
                         const int* positions, const int* tok_seq, const int* slots, int* last_token, int num_tokens,

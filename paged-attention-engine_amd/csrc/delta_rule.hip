@@ -21,8 +21,8 @@
 // per head (`channel_decay`: the decay's input and dt_bias are then H x D wide and row d of a head's S is
 // multiplied by its own number); beta, the decay's input and the gate read from rows of their own instead of
 // the projected rows' tail (a design whose decay and gate pass through a narrow product first); sigmoid
-// instead of SiLU on the gate.  The recurrence kernels also run a matrix memory that only adds
-// (`delta` off: u = beta v, nothing is read back before the write; see matrix_memory.hip).
+// instead of SiLU on the gate.  The recurrence kernels also run a state that only adds, with a decay per key
+// channel (`delta` off: u = beta v, nothing is read back before the write; see linear_attention.hip).
 //
 // Everything but the projected rows is float32: the convolution's sums, the unit vectors, beta,
 // the decay and its logarithm, the state, the read-out and the norm.  The order in which a
@@ -388,7 +388,7 @@ void pae_launch_recurrence(const float* q, const float* k, const float* v, const
                            int D, int V, int num_seqs, int channel_decay, int delta, float* o, hipStream_t stream);
 
 // The recurrence over a step's rows for every (sequence, head, column of S).  `channel_decay`: `decay` is
-// [T][H][D] instead of [T][H]; `delta` off: u = beta v (a memory that only adds).
+// [T][H][D] instead of [T][H]; `delta` off: u = beta v (a state that only adds; with `channel_decay` only).
 void pae_launch_recurrence(const float* q, const float* k, const float* v, const float* beta, const float* decay,
                            const int4* runs, const int* slots, float* state, int64_t state_slot_stride, int G, int H,
                            int D, int V, int num_seqs, int channel_decay, int delta, float* o, hipStream_t stream) {
@@ -401,8 +401,7 @@ void pae_launch_recurrence(const float* q, const float* k, const float* v, const
   do {                                                        \
     if (channel_decay && delta) GROUP_AS(R, L, CH, true, true);      \
     else if (channel_decay) GROUP_AS(R, L, CH, true, false);  \
-    else if (delta) GROUP_AS(R, L, CH, false, true);          \
-    else GROUP_AS(R, L, CH, false, false);                    \
+    else GROUP_AS(R, L, CH, false, true);                     \
   } while (0)
   if (D <= 16) GROUP(4, 4, 32);
   else if (D <= 32) GROUP(8, 4, 32);

@@ -19,41 +19,9 @@
 // projected rows and the result are in the activation type.  A decay of 1, 0 or above 1 needs no special case.
 #include "common.h"
 #include "api.h"
-
-typedef __attribute__((ext_vector_type(4))) float f32x4;
+#include "recurrent_device.h"
 
 #define FD_VS 64  // value features of a workgroup in the chunk kernels
-
-__device__ __forceinline__ float fd_act(float z, int silu) { return silu ? z / (1.0f + expf(-z)) : z; }
-
-// four numbers of a projected row from feature i on (those at or beyond `end` are zero), activated
-template <typename T>
-__device__ __forceinline__ void fd_load4(const T* row, int i, int end, bool vec, int silu, float (&v)[4]) {
-  if (vec && i + 4 <= end) {
-    if (sizeof(T) == 4) {
-      const float4 x = *reinterpret_cast<const float4*>((const float*)row + i);
-      v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w;
-    } else {
-      const uint2 x = *reinterpret_cast<const uint2*>((const bf16_t*)row + i);  // a bfloat16 is the upper half of a float
-      v[0] = __uint_as_float(x.x << 16); v[1] = __uint_as_float(x.x & 0xffff0000u);
-      v[2] = __uint_as_float(x.y << 16); v[3] = __uint_as_float(x.y & 0xffff0000u);
-    }
-  } else {
-#pragma unroll
-    for (int e = 0; e < 4; ++e) v[e] = i + e < end ? to_f32(row[i + e]) : 0.f;
-  }
-#pragma unroll
-  for (int e = 0; e < 4; ++e) v[e] = fd_act(v[e], silu);  // SiLU of 0 is 0
-}
-
-// Sum over 16 neighbouring lanes, in every one of them.
-__device__ __forceinline__ float fd_sum16(float v) {
-  v += __shfl_xor(v, 8, 16);
-  v += __shfl_xor(v, 4, 16);
-  v += __shfl_xor(v, 2, 16);
-  v += __shfl_xor(v, 1, 16);
-  return v;
-}
 
 // ---------------------------------------------------------------------------------------------- serial
 // runs[i] = (table row of the sequence, first flat row, rows, unused).  One workgroup per (run, head, 16 columns of S);
@@ -95,13 +63,13 @@ __global__ __launch_bounds__(256) void fixed_decay_serial_kernel(const T* __rest
       const int which = e / (DP / 4), d = e % (DP / 4) * 4, i = which / 2;
       const T* row = proj + (int64_t)(run.y + first + i) * row_stride + ((which % 2) * H + h) * (int64_t)D;
       float x[4];
-      fd_load4(row, d, D, rows_vec, silu, x);
+      load_row4(row, d, D, rows_vec, silu, x);
       *reinterpret_cast<float4*>((which % 2 ? s_k : s_q) + i * DP + d) = make_float4(x[0], x[1], x[2], x[3]);
     }
     float v[FD_STEPS];
 #pragma unroll
     for (int i = 0; i < FD_STEPS; ++i)
-      v[i] = i < n && live ? fd_act(to_f32(proj[(int64_t)(run.y + first + i) * row_stride + 2 * H * (int64_t)D + h * V + col]), silu) : 0.f;
+      v[i] = i < n && live ? recurrent_act(to_f32(proj[(int64_t)(run.y + first + i) * row_stride + 2 * H * (int64_t)D + h * V + col]), silu) : 0.f;
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < FD_STEPS; ++i) {
@@ -116,7 +84,7 @@ __global__ __launch_bounds__(256) void fixed_decay_serial_kernel(const T* __rest
         S[r][2] = fmaf(k4.z, v[i], decay * S[r][2]); o = fmaf(S[r][2], q4.z, o);
         S[r][3] = fmaf(k4.w, v[i], decay * S[r][3]); o = fmaf(S[r][3], q4.w, o);
       }
-      o = fd_sum16(o);
+      o = sum16(o);
       if (live && sub == 0) out[((int64_t)(run.y + first + i) * H + h) * V + col] = o;
     }
   }
@@ -155,7 +123,7 @@ __global__ __launch_bounds__(C * 4) void fixed_decay_chunk_sums_kernel(const T* 
     const int j = e / (DT * 4), d = e % (DT * 4) * 4;
     float x[4] = {0.f, 0.f, 0.f, 0.f};
     if (j < n) {
-      fd_load4(proj + (int64_t)(chunk.y + j) * row_stride + (H + h) * (int64_t)D, d, D, kvec, silu, x);
+      load_row4(proj + (int64_t)(chunk.y + j) * row_stride + (H + h) * (int64_t)D, d, D, kvec, silu, x);
       const float w = pw[n - 1 - j];
 #pragma unroll
       for (int i = 0; i < 4; ++i) x[i] *= w;
@@ -166,7 +134,7 @@ __global__ __launch_bounds__(C * 4) void fixed_decay_chunk_sums_kernel(const T* 
     const int j = e / (FD_VS / 4), v = e % (FD_VS / 4) * 4;
     float x[4] = {0.f, 0.f, 0.f, 0.f};
     if (j < n && v0 + v < V)
-      fd_load4(proj + (int64_t)(chunk.y + j) * row_stride + 2 * H * (int64_t)D + h * V, v0 + v, V, vvec, silu, x);
+      load_row4(proj + (int64_t)(chunk.y + j) * row_stride + 2 * H * (int64_t)D + h * V, v0 + v, V, vvec, silu, x);
     *reinterpret_cast<float4*>(s_v + j * VST + v) = make_float4(x[0], x[1], x[2], x[3]);
   }
   __syncthreads();
@@ -252,19 +220,19 @@ __global__ __launch_bounds__(C * 4) void fixed_decay_chunk_out_kernel(const T* _
   for (int s = 0; s < DT; ++s) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) q[s][i] = 0.f;
-    if (query < n) fd_load4(proj + (int64_t)(chunk.y + query) * row_stride + h * (int64_t)D, 16 * s + 4 * g4, D, kvec, silu, q[s]);
+    if (query < n) load_row4(proj + (int64_t)(chunk.y + query) * row_stride + h * (int64_t)D, 16 * s + 4 * g4, D, kvec, silu, q[s]);
   }
   for (int e = threadIdx.x; e < C * DT * 4; e += NT) {
     const int j = e / (DT * 4), d = e % (DT * 4) * 4;
     float x[4] = {0.f, 0.f, 0.f, 0.f};
-    if (j < n) fd_load4(proj + (int64_t)(chunk.y + j) * row_stride + (H + h) * (int64_t)D, d, D, kvec, silu, x);
+    if (j < n) load_row4(proj + (int64_t)(chunk.y + j) * row_stride + (H + h) * (int64_t)D, d, D, kvec, silu, x);
     *reinterpret_cast<float4*>(s_k + j * DS + d) = make_float4(x[0], x[1], x[2], x[3]);
   }
   for (int e = threadIdx.x; e < C * (FD_VS / 4); e += NT) {
     const int j = e / (FD_VS / 4), v = e % (FD_VS / 4) * 4;
     float x[4] = {0.f, 0.f, 0.f, 0.f};
     if (j < n && v0 + v < V)
-      fd_load4(proj + (int64_t)(chunk.y + j) * row_stride + 2 * H * (int64_t)D + h * V, v0 + v, V, vvec, silu, x);
+      load_row4(proj + (int64_t)(chunk.y + j) * row_stride + 2 * H * (int64_t)D + h * V, v0 + v, V, vvec, silu, x);
     *reinterpret_cast<float4*>(s_v + j * VST + v) = make_float4(x[0], x[1], x[2], x[3]);
   }
   if (threadIdx.x <= C) s_pw[threadIdx.x] = powers[(int64_t)h * (C + 1) + threadIdx.x];
@@ -367,7 +335,7 @@ __global__ __launch_bounds__(256) void row_norm_gate_kernel(const float* __restr
   for (int i = threadIdx.x * W; i < N; i += 256 * W) {
     float z[4], r[4];
     if (VEC) {
-      fd_load4(gate, i, N, true, 0, z);
+      load_row4(gate, i, N, true, 0, z);
       const float4 a = *reinterpret_cast<const float4*>(row + i);
       r[0] = a.x; r[1] = a.y; r[2] = a.z; r[3] = a.w;
     } else {

@@ -96,7 +96,9 @@ def _declare(lib) -> None:
         "pae_activation": [I, P, L, I, P, I, I, P],
         "pae_delta_rule_step": [I, P, L, I, I, P, P, P, P, P, P, L, I, I, I, I, I, P, P, F, P, L, P, I, F, P, P,
                                 P, L, I, P, L, P, L, I, P],
-        "pae_matrix_memory_step": [I, P, L, P, L, P, I, I, P, P, I, I, I, F, P, L, P, L, P, I, F, F, P, P, P],
+        "pae_matrix_memory_step": [I, P, L, P, L, P, P, L, P, P, I, I, P, I, P, I, P, I, P, I, I, I, F, P, L, P, L, P, I, F, F, P,
+                                   P, P],
+        "pae_matrix_memory_chunk": [I],
         "pae_embedding_pairs": [I, P, P, P, P, P, P, P, P, I, I, I, F, I, I, I, P],
         "pae_sum_norm2": [I, P, I, P, P, P, P, P, P, I, P, I, F, P, P, P, I, I, I, P],
         "pae_project_f32": [I, P, L, P, L, P, P, I, I, I, I, P],
@@ -150,7 +152,7 @@ def _declare(lib) -> None:
     lib.pae_skinny_ticket_floats.restype = c_int64
     lib.pae_delta_rule_work_floats.argtypes = [I, I, I, I, I, I]
     lib.pae_delta_rule_work_floats.restype = c_int64
-    lib.pae_matrix_memory_work_floats.argtypes = [I, I, I, I]
+    lib.pae_matrix_memory_work_floats.argtypes = [I, I, I, I, I]
     lib.pae_matrix_memory_work_floats.restype = c_int64
     lib.pae_linear_attention_work_floats.argtypes = [I, I, I, I]
     lib.pae_linear_attention_work_floats.restype = c_int64
@@ -1544,37 +1546,56 @@ def delta_rule_step(proj: torch.Tensor, out: torch.Tensor, tok_seq: torch.Tensor
         1 if channel_decay else 0, _stream()))
 
 
-def matrix_memory_step(proj: torch.Tensor, gate: torch.Tensor, gate_logits: torch.Tensor, out: torch.Tensor,
-                       seq_runs: torch.Tensor, slots: torch.Tensor, state: torch.Tensor, maximum: torch.Tensor,
-                       norm_w: torch.Tensor, H: int, D: int, V: int, gate_cap: float, norm_eps: float,
-                       floor_eps: float) -> None:
+def matrix_memory_chunk(key_dim: int) -> int:
+    """Tokens a chunk of `matrix_memory_step` holds for that key width; 0: its runs of any length go token by token."""
+    return library().pae_matrix_memory_chunk(int(key_dim))
+
+
+def matrix_memory_step(proj: torch.Tensor, gate: torch.Tensor, gate_logits: Optional[torch.Tensor], out: torch.Tensor,
+                       serial: torch.Tensor, chunks: torch.Tensor, scans: torch.Tensor, slots: torch.Tensor,
+                       state: torch.Tensor, maximum: torch.Tensor, norm_w: torch.Tensor, H: int, D: int, V: int,
+                       gate_cap: float, norm_eps: float, floor_eps: float, gates_from=None) -> None:
     """A matrix memory with exponential gates over a step's rows.  `proj` [T, >= 2HD + HV] holds per token
     [q | k | v]; `gate` [T, HV] (a view of rows in proj's type) is the output gate's input; `gate_logits` float32
-    [T, 2H] the input and forget gates' sums with their biases.  `state` float32 [slots, H, V + 1, D] (the
+    [T, 2H] the input and forget gates' sums with their biases, or None in a step without chunks, and `gates_from` =
+    (x [T, K], weight [2H, K], bias float32 [2H]) what they are then formed from.  The step's runs of tokens are in
+    three int32 lists of rows of four as for `fixed_decay_step`: `serial`, `chunks` (up to `matrix_memory_chunk(D)`
+    rows each) and `scans`.  `state` float32 [slots, H, V + 1, D] (the
     memory, and as its last column the sum of gated keys) and `maximum` float32 [slots, H] are the requests'
     state, read and moved on; `out` [T, H * V] receives o / (max(|n . q|, exp(-m)) + floor_eps), normed over V,
     times `norm_w` [H * V] and sigmoid(gate), in proj's type."""
     _not_while_recording("matrix_memory_step")
-    _gpu(proj, gate, gate_logits, out, seq_runs, slots, state, maximum, norm_w)
-    T, S = proj.shape[0], seq_runs.shape[0]
+    _gpu(proj, gate, gate_logits, out, serial, chunks, scans, slots, state, maximum, norm_w)
+    T = proj.shape[0]
     assert proj.dim() == 2 and proj.stride(1) == 1 and proj.shape[1] >= 2 * H * D + H * V
     assert gate.shape == (T, H * V) and gate.stride(1) == 1 and gate.dtype == proj.dtype
-    assert gate_logits.dtype == torch.float32 and gate_logits.shape == (T, 2 * H) and gate_logits.is_contiguous()
+    x = gate_w = gate_b = None
+    if gate_logits is not None:
+        assert gate_logits.dtype == torch.float32 and gate_logits.shape == (T, 2 * H) and gate_logits.is_contiguous()
+    else:
+        x, gate_w, gate_b = gates_from
+        _gpu(x, gate_w, gate_b)
+        assert chunks.shape[0] == 0, "runs in chunks take the gates' sums, not what they are formed from"
+        assert x.dim() == 2 and x.shape[0] == T and x.stride(1) == 1 and x.dtype == gate_w.dtype == proj.dtype
+        assert gate_w.shape == (2 * H, x.shape[1]) and gate_w.is_contiguous()
+        assert gate_b.dtype == torch.float32 and gate_b.numel() == 2 * H and gate_b.is_contiguous()
     assert out.shape == (T, H * V) and out.is_contiguous() and out.dtype == proj.dtype
-    assert slots.dtype == torch.int32 and slots.numel() >= S and slots.is_contiguous()
-    assert seq_runs.dtype == torch.int32 and seq_runs.shape == (S, 4) and seq_runs.is_contiguous()
-    assert seq_runs.data_ptr() % 16 == 0
+    for lists in (serial, chunks, scans):
+        assert lists.dtype == torch.int32 and lists.dim() == 2 and lists.shape[1] == 4 and lists.is_contiguous()
+        assert lists.numel() == 0 or lists.data_ptr() % 16 == 0
+    assert slots.dtype == torch.int32 and slots.is_contiguous()
     assert state.dtype == torch.float32 and tuple(state.shape[1:]) == (H, V + 1, D) and state[0].is_contiguous()
     assert maximum.dtype == torch.float32 and tuple(maximum.shape[1:]) == (H,) and maximum.stride(1) == 1
     assert maximum.shape[0] == state.shape[0] and norm_w.numel() == H * V and norm_w.is_contiguous()
     wp, wf = _param(norm_w)
     lib = library()
-    work = torch.empty(lib.pae_matrix_memory_work_floats(T, H, D, V), dtype=torch.float32, device=proj.device)
+    work = torch.empty(lib.pae_matrix_memory_work_floats(T, chunks.shape[0], H, D, V), dtype=torch.float32, device=proj.device)
     _check(lib.pae_matrix_memory_step(
-        code_of(proj.dtype), proj.data_ptr(), proj.stride(0), gate.data_ptr(), gate.stride(0), gate_logits.data_ptr(), T, S,
-        seq_runs.data_ptr(), slots.data_ptr(), H, D, V, float(gate_cap), state.data_ptr(), state.stride(0),
-        maximum.data_ptr(), maximum.stride(0), wp, wf, float(norm_eps), float(floor_eps), work.data_ptr(), out.data_ptr(),
-        _stream()))
+        code_of(proj.dtype), proj.data_ptr(), proj.stride(0), gate.data_ptr(), gate.stride(0), _ptr(gate_logits), _ptr(x),
+        x.stride(0) if x is not None else 0, _ptr(gate_w), _ptr(gate_b), x.shape[1] if x is not None else 0, T,
+        serial.data_ptr(), serial.shape[0], chunks.data_ptr(), chunks.shape[0], scans.data_ptr(), scans.shape[0],
+        slots.data_ptr(), H, D, V, float(gate_cap), state.data_ptr(), state.stride(0), maximum.data_ptr(), maximum.stride(0),
+        wp, wf, float(norm_eps), float(floor_eps), work.data_ptr(), out.data_ptr(), _stream()))
 
 
 def embedding_pairs(out: torch.Tensor, table: torch.Tensor, pairs: torch.Tensor, ids: torch.Tensor, positions: torch.Tensor,

@@ -42,6 +42,28 @@ def sequence_runs(shape: StepShape):
                       for x in (start, n, past, 0)], 4)}
 
 
+SERIAL_ROWS = 16  # runs of up to this many tokens walk a recurrence token by token, longer ones go in chunks
+
+
+def runs_and_chunks_key(chunk: int):
+    return ("runs token by token and in chunks", chunk)
+
+
+def runs_and_chunks(shape: StepShape, chunk: int):
+    """Work lists of the recurrent kernels that take longer runs in chunks of `chunk` tokens (0: no chunks), see
+    `kernels.lib.fixed_decay_step`."""
+    serial, chunks, scans = [], [], []
+    for row, (start, n) in enumerate(zip(shape.q_starts, shape.q_lens)):
+        if n <= SERIAL_ROWS or not chunk:
+            serial += [row, start, n, 0]
+            continue
+        first = len(chunks) // 4
+        for at in range(0, n, chunk):
+            chunks += [row, start + at, min(chunk, n - at), 0]
+        scans += [row, first, len(chunks) // 4 - first, n - (n - 1) // chunk * chunk]
+    return {"serial": (serial, 4), "chunks": (chunks, 4), "scans": (scans, 4)}
+
+
 @register_mixer("gated_delta")
 class GatedDeltaMixer(Part):
     graph_safe = True

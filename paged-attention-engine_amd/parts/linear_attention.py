@@ -28,7 +28,7 @@ import torch
 from ..cache.manager import StateSpec
 from ..kernels import lib as K
 from .base import Part, ScaleShape, StepShape, plain_rows, register_mixer
-from .delta import SEQ_RUNS, sequence_runs
+from .delta import SEQ_RUNS, runs_and_chunks, runs_and_chunks_key, sequence_runs
 from .linear import Linear, rows_a_graph_may_hold
 
 
@@ -115,23 +115,6 @@ class GatedLinearAttention(Part):
         return self.out.branch(out, ctx.sink)
 
 
-SERIAL_ROWS = 16  # runs of up to this many tokens walk the recurrence token by token, longer ones go in chunks
-
-
-def decay_runs(shape: StepShape, chunk: int):
-    """Work lists of `kernels.lib.fixed_decay_step` for chunks of `chunk` tokens (0: no chunks)."""
-    serial, chunks, scans = [], [], []
-    for row, (start, n) in enumerate(zip(shape.q_starts, shape.q_lens)):
-        if n <= SERIAL_ROWS or not chunk:
-            serial += [row, start, n, 0]
-            continue
-        first = len(chunks) // 4
-        for at in range(0, n, chunk):
-            chunks += [row, start + at, min(chunk, n - at), 0]
-        scans += [row, first, len(chunks) // 4 - first, n - (n - 1) // chunk * chunk]
-    return {"serial": (serial, 4), "chunks": (chunks, 4), "scans": (scans, 4)}
-
-
 @register_mixer("fixed_decay_linear_attention")
 class FixedDecayAttention(Part):
     """Lightning attention: per token q = act(W_q h) and k = act(W_k h) (H heads of D), v = act(W_v h) (H heads of V),
@@ -172,10 +155,10 @@ class FixedDecayAttention(Part):
         return K.fixed_decay_chunk(self.spec.key_dim)
 
     def step_lists_key(self, block_size: int):
-        return ("runs under a fixed decay", self.chunk)
+        return runs_and_chunks_key(self.chunk)
 
     def step_lists(self, shape: StepShape):
-        return decay_runs(shape, self.chunk)
+        return runs_and_chunks(shape, self.chunk)
 
     def _projections(self):
         s = self.spec

@@ -13,11 +13,12 @@ Each head's o is divided by its root mean square over V, multiplied by a weight 
 and by sigmoid(W_g h), and projected out by W_o.
 
 q, k, v and the output gate are one product over concatenated weights; the two gates' sums are formed in
-float32 by a product of their own (their logarithms add up over a sequence, so they do not pass the
-activation type).  The state lives in the cache manager's per-request slots as two named float32 tensors,
+float32 by themselves (their logarithms add up over a sequence, so they do not pass the activation type): by a
+product of their own in steps with runs in chunks, inside the kernel that forms the gates in all others.  The state lives in the cache manager's per-request slots as two named float32 tensors,
 "memory" [H, V + 1, D] (column V holds n: it is the memory's column for a value that is always 1) and
 "memory_max" [H]; a slot is zeroed when a request takes it, which is the design's start state.  Everything
-after the projections is float32 inside `kernels.lib.matrix_memory_step`.  Nothing is kept per token.
+after the projections is float32 inside `kernels.lib.matrix_memory_step`, which takes short runs token by token and
+longer ones in chunks.  Nothing is kept per token.
 """
 
 from __future__ import annotations
@@ -27,7 +28,7 @@ import torch
 from ..cache.manager import StateSpec
 from ..kernels import lib as K
 from .base import Part, ScaleShape, StepShape, plain_rows, register_mixer
-from .delta import SEQ_RUNS, sequence_runs
+from .delta import runs_and_chunks, runs_and_chunks_key
 from .linear import Linear, rows_a_graph_may_hold
 
 
@@ -54,11 +55,15 @@ class MatrixMemory(Part):
         return (StateSpec((s.num_heads, s.value_dim + 1, s.key_dim), torch.float32, "memory"),
                 StateSpec((s.num_heads,), torch.float32, "memory_max"))
 
+    @property
+    def chunk(self) -> int:
+        return K.matrix_memory_chunk(self.spec.key_dim)
+
     def step_lists_key(self, block_size: int):
-        return SEQ_RUNS
+        return runs_and_chunks_key(self.chunk)
 
     def step_lists(self, shape: StepShape):
-        return sequence_runs(shape)
+        return runs_and_chunks(shape, self.chunk)
 
     def _projections(self):
         """(name, rows) of the projections that share one product, in the order of its columns."""
@@ -95,10 +100,12 @@ class MatrixMemory(Part):
         x = plain_rows(x)
         H, D, V = s.num_heads, s.key_dim, s.value_dim
         proj = self.proj(x)
-        gate_logits = K.project_f32(x, self.gate_weight, self.gate_bias)
+        lists = ctx.memo[self.step_lists_key(ctx.cache.block_size)]
+        in_chunks = lists["chunks"].shape[0] > 0
+        gate_logits = K.project_f32(x, self.gate_weight, self.gate_bias) if in_chunks else None
         state = ctx.cache.state_of(ctx.cache_entry)
         out = torch.empty((x.shape[0], H * V), dtype=x.dtype, device=x.device)
-        K.matrix_memory_step(proj, proj[:, 2 * H * D + H * V:], gate_logits, out, ctx.memo[SEQ_RUNS]["runs"], ctx.slots,
-                             state["memory"], state["memory_max"], self.norm, H, D, V, s.gate_cap, s.norm_eps,
-                             s.readout_floor)
+        K.matrix_memory_step(proj, proj[:, 2 * H * D + H * V:], gate_logits, out, lists["serial"], lists["chunks"],
+                             lists["scans"], ctx.slots, state["memory"], state["memory_max"], self.norm, H, D, V, s.gate_cap,
+                             s.norm_eps, s.readout_floor, gates_from=None if in_chunks else (x, self.gate_weight, self.gate_bias))
         return self.out.branch(out, ctx.sink)

@@ -138,15 +138,15 @@ def test_what_the_layers_keep():
 def test_work_lists_of_the_convolutions_and_the_recurrence():
     from paged_attention_engine_amd.parts import StepShape
     from paged_attention_engine_amd.parts.input_conv import conv_tiles
-    from paged_attention_engine_amd.parts.linear_attention import SERIAL_ROWS, decay_runs
+    from paged_attention_engine_amd.parts.delta import SERIAL_ROWS, runs_and_chunks
 
     shape = StepShape((7, 8, 9), (0, 1, 151), (1, 150, SERIAL_ROWS), (40, 5, 0), 16)
-    lists = decay_runs(shape, 64)
+    lists = runs_and_chunks(shape, 64)
     assert lists["serial"] == ([0, 0, 1, 0, 2, 151, SERIAL_ROWS, 0], 4)
     assert lists["chunks"] == ([1, 1, 64, 0, 1, 65, 64, 0, 1, 129, 22, 0], 4)
     assert lists["scans"] == ([1, 0, 3, 22], 4)
-    assert decay_runs(StepShape((7,), (0,), (128,), (0,), 16), 64)["scans"] == ([0, 0, 2, 64], 4)  # a whole last chunk
-    assert decay_runs(shape, 0) == {"serial": ([0, 0, 1, 0, 1, 1, 150, 0, 2, 151, SERIAL_ROWS, 0], 4), "chunks": ([], 4), "scans": ([], 4)}
+    assert runs_and_chunks(StepShape((7,), (0,), (128,), (0,), 16), 64)["scans"] == ([0, 0, 2, 64], 4)  # a whole last chunk
+    assert runs_and_chunks(shape, 0) == {"serial": ([0, 0, 1, 0, 1, 1, 150, 0, 2, 151, SERIAL_ROWS, 0], 4), "chunks": ([], 4), "scans": ([], 4)}
     lists = conv_tiles(StepShape((7, 8), (0, 3), (3, 10), (40, 5), 16), 8)
     assert lists["tiles"] == ([0, 0, 3, 0, 1, 3, 8, 0, 1, 11, 2, 8], 4)
     assert lists["runs"] == ([0, 3, 40, 0, 3, 10, 5, 0], 4)

@@ -103,6 +103,15 @@ def test_terms_join_the_stream_and_both_norms_read_it(dtype, H):
 # ----------------------------------------------------------------------------- matrix memory
 
 
+def memory_lists(n, D):
+    """The work lists of one run of `n` tokens: token by token, chunks, runs in chunks."""
+    from paged_attention_engine_amd.parts.base import StepShape
+    from paged_attention_engine_amd.parts.delta import runs_and_chunks
+
+    lists = runs_and_chunks(StepShape((0,), (0,), (n,), (0,), 16), K().matrix_memory_chunk(D))
+    return [torch.tensor(lists[name][0], dtype=torch.int32, device=DEV).view(-1, 4) for name in ("serial", "chunks", "scans")]
+
+
 def memory_inputs(gen, T, H, D, V, dtype, cap):
     proj = (torch.randn((T, 2 * H * D + 2 * H * V), generator=gen) * 0.7).to(dtype)
     logits = torch.randn((T, 2 * H), generator=gen) * 3.0
@@ -146,7 +155,7 @@ def test_matrix_memory_whole_and_in_steps_in_used_slots(dtype, shape):
             out = torch.empty((n, H * V), dtype=dtype, device=DEV)
             piece = proj[p:p + n].to(DEV)
             K().matrix_memory_step(piece, piece[:, 2 * H * D + H * V:], logits[p:p + n].contiguous().to(DEV), out,
-                                   runs_of([n], [p]), slots, state, top, norm.to(DEV), H, D, V, cap, eps, 1e-6)
+                                   *memory_lists(n, D), slots, state, top, norm.to(DEV), H, D, V, cap, eps, 1e-6)
             rows.append(out)
             p += n
         close(torch.cat(rows), want, rel, f"memory {shape} cut {cuts[:2]}")
@@ -166,7 +175,7 @@ def test_matrix_memory_keeps_what_it_was_told_to():
     state, top = torch.zeros((1, 1, V + 1, D), device=DEV), torch.zeros((1, 1), device=DEV)
     out = torch.empty((T, V), device=DEV)
     piece = proj.to(DEV)
-    K().matrix_memory_step(piece, piece[:, 2 * D + V:], logits.to(DEV), out, runs_of([T], [0]),
+    K().matrix_memory_step(piece, piece[:, 2 * D + V:], logits.to(DEV), out, *memory_lists(T, D),
                            torch.zeros(1, dtype=torch.int32, device=DEV), state, top, torch.ones(V, device=DEV), H, D, V, cap, 1e-6, 1e-6)
     close(out, want, 2e-5, "recall")
     v40 = proj[40, 2 * D:2 * D + V].double()

@@ -143,10 +143,10 @@ def decay_plain(proj, gate, norm, decays, H, D, V, eps):
 
 def decay_step(lib, proj, norm, decays, H, D, V, eps, lens, slots, state):
     """`proj` [rows, 2HD + 2HV] = [q | k | v | gate] of the sequences `lens` one after the other."""
-    from paged_attention_engine_amd.parts.linear_attention import decay_runs
+    from paged_attention_engine_amd.parts.delta import runs_and_chunks
 
     chunk = lib.fixed_decay_chunk(D)
-    lists = decay_runs(step_shape(lens, [0] * len(lens)), chunk)
+    lists = runs_and_chunks(step_shape(lens, [0] * len(lens)), chunk)
     powers = torch.pow(torch.tensor(decays, dtype=torch.float64)[:, None], torch.arange((chunk or 1) + 1, dtype=torch.float64))
     p = proj.to(DEV)
     out = torch.empty((proj.shape[0], H * V), dtype=proj.dtype, device=DEV)

@@ -188,11 +188,30 @@ def getodra_shape(shape: dict, layers: int) -> dict:
             "canon": {"taps": 4}, "layers": out}
 
 
+def mulenex_shape(shape: dict, layers: int) -> dict:
+    """A Mulenex configuration with the layer sizes of the Qwen2.5 shape `shape`: the same width, head counts, head size and
+    vocabulary; in turn attention (values as wide as keys, per-head norms, capped scores, a query temperature, mixed
+    values, a gate per head) and a matrix memory with as many heads of the same size; feed-forwards in turn dense, of
+    the shape's width, and routed, 32 experts of a quarter of that width with three a token beside a shared one as
+    wide, so that a token's routed feed-forward is as wide as the dense one."""
+    heads, kv, hd = shape["num_attention_heads"], shape["num_key_value_heads"], shape["head_dim"]
+    attention = {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv, "dim": hd, "vdim": hd, "scale": hd ** -0.5,
+                                                "softcap": 50.0, "q_temp": {"coef": 0.1, "every": 8192}, "v_mix": True}}
+    memory = {"type": "mlstm", "mixer": {"heads": heads, "dim": hd, "vdim": hd, "gate_cap": 15.0}}
+    dense = {"kind": "dense", "ff": shape["intermediate_size"]}
+    ff = shape["intermediate_size"] // 4 // 8 * 8
+    moe = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": 32, "top": 3}, "shared": {"ff": ff}}
+    mlps = [dense, moe, moe, dense]
+    return {"architecture": "Mulenex", "vocab": shape["vocab_size"], "width": shape["hidden_size"],
+            "norm": {"eps": shape["rms_norm_eps"]},
+            "layers": [dict(memory if i % 2 else attention, mlp=mlps[i % 4]) for i in range(layers)]}
+
+
 def design_run(args, shape: dict) -> int:
-    """`--design danonex|ritalorn|dagavik|zikezen|getodra`: decode steps (batch 1, 8, 64 at the context asked for) and prefills of
+    """`--design danonex|ritalorn|dagavik|zikezen|getodra|mulenex`: decode steps (batch 1, 8, 64 at the context asked for) and prefills of
     2,048 and 8,192 tokens of a model of that design with the shape's layer sizes, and beside each the same
     measurement of the Qwen2.5 shape (and, for ritalorn and dagavik, of the Danonex shape; for zikezen, of the Dagavik
-    shape; for getodra, of the Ritalorn and Zikezen shapes) with the same number of layers (for zikezen: of layer runs).  One JSON line."""
+    shape; for getodra, of the Ritalorn and Zikezen shapes; for mulenex, of the Dagavik and Zikezen shapes) with the same number of layers (for zikezen: of layer runs).  One JSON line."""
     import torch
 
     layers = args.layers or 8
@@ -201,7 +220,12 @@ def design_run(args, shape: dict) -> int:
                         f"prefill tok/s", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
               "dtype": "bf16" if args.dtype == "bfloat16" else "fp32", "context": args.ctx,
               "data": "synthetic: seeded uniform token ids, random weights N(0, 0.02)", "designs": {}}
-    if args.design == "getodra":
+    if args.design == "mulenex":
+        configs = {"mulenex": mulenex_shape(shape, layers)}
+        if not args.alone:
+            configs.update({"dagavik": dagavik_shape(shape, layers), "zikezen": zikezen_shape(shape, layers),
+                            "qwen2": dict(shape, num_hidden_layers=layers)})
+    elif args.design == "getodra":
         configs = {"getodra": getodra_shape(shape, layers)}
         if not args.alone:
             configs.update({"ritalorn": ritalorn_shape(shape, layers), "zikezen": zikezen_shape(shape, layers),
@@ -468,12 +492,12 @@ def main() -> int:
     parser.add_argument("--dtype", choices=("bfloat16", "float32"), default="bfloat16")
     parser.add_argument("--no-points", action="store_true", help="skip the batch 1 / 64 and prefill runs")
     parser.add_argument("--prefill-only", action="store_true", help="time the 2,048-token prefill alone (for profiles)")
-    parser.add_argument("--design", choices=("qwen2", "danonex", "ritalorn", "dagavik", "zikezen", "getodra"), default="qwen2",
-                        help="danonex, ritalorn, dagavik, zikezen, getodra: a model of that design with the shape's layer sizes (8 layers "
+    parser.add_argument("--design", choices=("qwen2", "danonex", "ritalorn", "dagavik", "zikezen", "getodra", "mulenex"), default="qwen2",
+                        help="danonex, ritalorn, dagavik, zikezen, getodra, mulenex: a model of that design with the shape's layer sizes (8 layers "
                              "unless --layers says otherwise) beside the Qwen2.5 shape (ritalorn, dagavik: and the Danonex shape; "
-                             "zikezen: and the Dagavik shape; getodra: and the Ritalorn and Zikezen shapes) with as many layers: "
+                             "zikezen: and the Dagavik shape; getodra: and the Ritalorn and Zikezen shapes; mulenex: and the Dagavik and Zikezen shapes) with as many layers: "
                              "decode at batch 1, 8, 64 and prefills of 2,048 and 8,192 tokens")
-    parser.add_argument("--alone", action="store_true", help="with --design ritalorn, dagavik, zikezen or getodra: that design only (for profiles)")
+    parser.add_argument("--alone", action="store_true", help="with --design ritalorn, dagavik, zikezen, getodra or mulenex: that design only (for profiles)")
     args = parser.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU only: this engine has no multi-GPU path (run with --gpus 1)")
@@ -484,7 +508,7 @@ def main() -> int:
         print("bench.py needs a GPU", file=sys.stderr)
         return 1
     shape = QWEN25_1P5B if args.model == "1.5b" else OTHER_SHAPES[args.model]
-    if args.design in ("danonex", "ritalorn", "dagavik", "zikezen", "getodra"):
+    if args.design in ("danonex", "ritalorn", "dagavik", "zikezen", "getodra", "mulenex"):
         try:
             return design_run(args, shape)
         except (Refused, Unresolved) as err:

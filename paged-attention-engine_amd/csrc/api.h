@@ -156,8 +156,8 @@ int pae_sum_norm2(int dtype, float* residual, int num_terms, const void* const* 
                   int num_rows, int hidden, int write_residual, hipStream_t stream);
 // a sublayer's output joins the stream through the norm after it; the norm before the next sublayer: see sandwich_norm.hip
 int pae_norm_join(int dtype, float* residual, int num_terms, const void* const* term_ptr, const int* term_is_f32,
-                  const int* term_parts, const int64_t* term_part_stride, const float* term_scale, const void* w_out,
-                  int w_out_is_f32, float eps, const void* w_next, int w_next_is_f32, float eps_next, void* normed,
+                  const int* term_parts, const int64_t* term_part_stride, const int* term_one_row, const float* term_scale,
+                  const void* w_out, int w_out_is_f32, float eps, const void* w_next, int w_next_is_f32, float eps_next, void* normed,
                   void* rows, int num_rows, int hidden, hipStream_t stream);
 // gated linear attention over a step's projected rows: see linear_attention.hip
 int pae_linear_attention_step(int dtype, const void* proj, int64_t row_stride, const void* z_in, int64_t z_stride,

@@ -158,27 +158,40 @@ __global__ void activation_kernel(T* __restrict__ x, int64_t n, int kind, const 
   if (i < n) x[i] = from_f32<T>(act_of(to_f32(x[i]) + (bias ? load_param(bias, b_is_f32, i % width) : 0.f), kind));
 }
 
-// eight bfloat16 numbers a thread (one 16-byte load and store), for sizes (and widths, with a bias) that are
-// multiples of eight
-__global__ void activation_bf16x8_kernel(uint4* __restrict__ x, int64_t nvec, int kind, const void* __restrict__ bias,
-                                         int b_is_f32, int width) {
+// eight bfloat16 numbers a thread (one 16-byte load and store), for sizes that are multiples of eight
+__global__ void activation_bf16x8_kernel(uint4* __restrict__ x, int64_t nvec, int kind) {
   const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= nvec) return;
   uint4 v = x[i];
   unsigned* w = reinterpret_cast<unsigned*>(&v);
-  float b[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-  if (bias) {
-    const int first = (int)(8 * i % width);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) b[j] = load_param(bias, b_is_f32, first + j);
-  }
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
-    const bf16_t lo = __float2bfloat16(act_of(__uint_as_float(w[j] << 16) + b[2 * j], kind));
-    const bf16_t hi = __float2bfloat16(act_of(__uint_as_float(w[j] & 0xffff0000u) + b[2 * j + 1], kind));
+    const bf16_t lo = __float2bfloat16(act_of(__uint_as_float(w[j] << 16), kind));
+    const bf16_t hi = __float2bfloat16(act_of(__uint_as_float(w[j] & 0xffff0000u), kind));
     w[j] = (unsigned)*reinterpret_cast<const unsigned short*>(&lo) | ((unsigned)*reinterpret_cast<const unsigned short*>(&hi) << 16);
   }
   x[i] = v;
+}
+
+// The same with a bias: a thread has eight columns of several rows, its biases in registers.
+__global__ __launch_bounds__(256) void activation_bias_bf16x8_kernel(uint4* __restrict__ x, int rows, int row_vecs, int kind,
+                                                                     const void* __restrict__ bias, int b_is_f32) {
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= row_vecs) return;
+  float b[8];
+#pragma unroll
+  for (int j = 0; j < 8; ++j) b[j] = load_param(bias, b_is_f32, 8 * c + j);
+  for (int r = blockIdx.y; r < rows; r += gridDim.y) {
+    uint4 v = x[(int64_t)r * row_vecs + c];
+    unsigned* w = reinterpret_cast<unsigned*>(&v);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const bf16_t lo = __float2bfloat16(act_of(__uint_as_float(w[j] << 16) + b[2 * j], kind));
+      const bf16_t hi = __float2bfloat16(act_of(__uint_as_float(w[j] & 0xffff0000u) + b[2 * j + 1], kind));
+      w[j] = (unsigned)*reinterpret_cast<const unsigned short*>(&lo) | ((unsigned)*reinterpret_cast<const unsigned short*>(&hi) << 16);
+    }
+    x[(int64_t)r * row_vecs + c] = v;
+  }
 }
 
 // x <- act(x + bias): rows of `width` numbers, bias (or null) one number per column
@@ -187,8 +200,14 @@ extern "C" int pae_activation(int dtype, void* x, int64_t n, int kind, const voi
   PAE_REQUIRE(!bias || (width > 0 && n % width == 0), "activation: %lld numbers are no rows of %d", (long long)n, width);
   PAE_REQUIRE(kind >= 0 && kind <= PAE_LAST_ACTIVATION, "activation: unknown kind %d", kind);
   if (n <= 0) return 0;
-  if (dtype == PAE_BF16 && n % 8 == 0 && (uintptr_t)x % 16 == 0 && (!bias || width % 8 == 0)) {
-    activation_bf16x8_kernel<<<(unsigned)((n / 8 + 255) / 256), 256, 0, stream>>>((uint4*)x, n / 8, kind, bias, b_is_f32, width);
+  if (dtype == PAE_BF16 && n % 8 == 0 && (uintptr_t)x % 16 == 0 && bias && width % 8 == 0) {
+    const int rows = (int)(n / width), row_vecs = width / 8;
+    activation_bias_bf16x8_kernel<<<dim3((row_vecs + 255) / 256, rows < 512 ? rows : 512), 256, 0, stream>>>((uint4*)x, rows, row_vecs,
+                                                                                                             kind, bias, b_is_f32);
+    return pae_check_launch("activation");
+  }
+  if (dtype == PAE_BF16 && n % 8 == 0 && (uintptr_t)x % 16 == 0 && !bias) {
+    activation_bf16x8_kernel<<<(unsigned)((n / 8 + 255) / 256), 256, 0, stream>>>((uint4*)x, n / 8, kind);
     return pae_check_launch("activation");
   }
   const unsigned blocks = (unsigned)((n + 255) / 256);

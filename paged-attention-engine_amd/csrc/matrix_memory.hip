@@ -516,8 +516,9 @@ __global__ __launch_bounds__(CH * 4) void memory_chunk_out_kernel(const T* __res
 }
 
 // ---------------------------------------------------------------------------------------------- division, norm, gate
-// A wavefront per (token, head), four heads a workgroup.
-template <typename T>
+// A wavefront per (token, head), four heads a workgroup; W features a lane at a time (2: all rows start on even features
+// of rows aligned for pairs).
+template <typename T, int W>
 __global__ __launch_bounds__(256) void memory_finish_kernel(const float* __restrict__ o, const float* __restrict__ nq,
                                                             const float* __restrict__ floors, const T* __restrict__ gates,
                                                             int64_t gate_stride, const void* __restrict__ weight, int w_is_f32,
@@ -528,16 +529,29 @@ __global__ __launch_bounds__(256) void memory_finish_kernel(const float* __restr
   const float* x = o + (t * H + h) * V;
   const float denom = fmaxf(fabsf(nq[t * H + h]), floors[t * H + h]) + floor_eps;
   float ss = 0.f;
-  for (int i = lane; i < V; i += PAE_WAVE) {
-    const float y = x[i] / denom;
-    ss = fmaf(y, y, ss);
+  struct alignas(W * sizeof(float)) Floats { float v[W]; };
+  struct alignas(W * sizeof(T)) Few { T v[W]; };
+  for (int i = lane * W; i < V; i += PAE_WAVE * W) {
+    const Floats a = *reinterpret_cast<const Floats*>(x + i);
+#pragma unroll
+    for (int e = 0; e < W; ++e) {
+      const float y = a.v[e] / denom;
+      ss = fmaf(y, y, ss);
+    }
   }
   ss = wave_sum(ss);
   const float inv = 1.0f / sqrtf(ss / (float)V + eps);
   const T* gate = gates + t * gate_stride + h * V;
-  for (int i = lane; i < V; i += PAE_WAVE) {
-    const float g = 1.0f / (1.0f + expf(-to_f32(gate[i])));
-    out[(t * H + h) * V + i] = from_f32<T>(x[i] / denom * inv * load_param(weight, w_is_f32, h * V + i) * g);
+  for (int i = lane * W; i < V; i += PAE_WAVE * W) {
+    const Floats a = *reinterpret_cast<const Floats*>(x + i);
+    const Few z = *reinterpret_cast<const Few*>(gate + i);
+    Few r;
+#pragma unroll
+    for (int e = 0; e < W; ++e) {
+      const float g = 1.0f / (1.0f + expf(-to_f32(z.v[e])));
+      r.v[e] = from_f32<T>(a.v[e] / denom * inv * load_param(weight, w_is_f32, h * V + i + e) * g);
+    }
+    *reinterpret_cast<Few*>(out + (t * H + h) * V + i) = r;
   }
 }
 
@@ -641,15 +655,21 @@ extern "C" int pae_matrix_memory_step(int dtype, const void* proj, int64_t row_s
   a.nq = rest;
   a.gates = MemoryGates{rest + TH, rest + 2 * TH, rest + 3 * TH, rest + 4 * TH, rest + 5 * TH, rest + 6 * TH};
   dim3 token_heads(num_tokens, (H + 3) / 4);
+  const int size = dtype == PAE_F32 ? 4 : 2;
+  const bool pairs = V % 2 == 0 && gate_stride % 2 == 0 && (uintptr_t)gate_in % (2 * size) == 0 && (uintptr_t)out % (2 * size) == 0;
+#define MEMORY_FINISH(T, W)                                                                                              \
+  memory_finish_kernel<T, W><<<token_heads, 256, 0, stream>>>(a.o, a.nq, a.gates.floors, (const T*)gate_in, gate_stride,  \
+                                                              norm_w, w_is_f32, norm_eps, floor_eps, H, V, (T*)out)
   if (dtype == PAE_F32) {
     memory_launch((const float*)proj, a, stream);
-    memory_finish_kernel<float><<<token_heads, 256, 0, stream>>>(a.o, a.nq, a.gates.floors, (const float*)gate_in, gate_stride,
-                                                                 norm_w, w_is_f32, norm_eps, floor_eps, H, V, (float*)out);
+    if (pairs) MEMORY_FINISH(float, 2);
+    else MEMORY_FINISH(float, 1);
   } else {
     memory_launch((const bf16_t*)proj, a, stream);
-    memory_finish_kernel<bf16_t><<<token_heads, 256, 0, stream>>>(a.o, a.nq, a.gates.floors, (const bf16_t*)gate_in, gate_stride,
-                                                                  norm_w, w_is_f32, norm_eps, floor_eps, H, V, (bf16_t*)out);
+    if (pairs) MEMORY_FINISH(bf16_t, 2);
+    else MEMORY_FINISH(bf16_t, 1);
   }
+#undef MEMORY_FINISH
   return pae_check_launch("matrix_memory_step");
 }
 

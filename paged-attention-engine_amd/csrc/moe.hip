@@ -91,6 +91,7 @@ extern "C" int pae_project_f32(int dtype, float* out, int64_t ldo, const void* A
 
 #define MOE_MAX_PER_LANE 16  // experts a lane holds: up to 1,024 experts
 
+template <int PER_LANE>
 __global__ __launch_bounds__(PAE_WAVE) void moe_route_kernel(const float* __restrict__ logits, int E, int groups, int keep,
                                                              int top, float scale, const float* __restrict__ choice_bias,
                                                              int64_t ldz, int among_chosen, int shared_pieces,
@@ -125,9 +126,9 @@ __global__ __launch_bounds__(PAE_WAVE) void moe_route_kernel(const float* __rest
   __syncthreads();
   // an expert may be chosen if fewer than `keep` groups come before its own (a larger score, or an equal one
   // at a lower index)
-  float mine[MOE_MAX_PER_LANE];
+  float mine[PER_LANE];
 #pragma unroll
-  for (int j = 0; j < MOE_MAX_PER_LANE; ++j) {
+  for (int j = 0; j < PER_LANE; ++j) {
     const int e = lane + PAE_WAVE * j;
     mine[j] = -INFINITY;
     if (e < E) {
@@ -143,7 +144,7 @@ __global__ __launch_bounds__(PAE_WAVE) void moe_route_kernel(const float* __rest
     float best = -INFINITY;
     int at = 0x7fffffff;
 #pragma unroll
-    for (int j = 0; j < MOE_MAX_PER_LANE; ++j)
+    for (int j = 0; j < PER_LANE; ++j)
       if (mine[j] > best) {  // a lane's experts ascend with j: the first of equals stays
         best = mine[j];
         at = lane + PAE_WAVE * j;
@@ -164,7 +165,7 @@ __global__ __launch_bounds__(PAE_WAVE) void moe_route_kernel(const float* __rest
       weights[t * places + r] = among_chosen ? expf(best - first) : score[at] / sum * scale;
     }
 #pragma unroll
-    for (int j = 0; j < MOE_MAX_PER_LANE; ++j)
+    for (int j = 0; j < PER_LANE; ++j)
       if (lane + PAE_WAVE * j == at) mine[j] = -INFINITY;
   }
   if (lane != 0) return;
@@ -189,8 +190,14 @@ extern "C" int pae_moe_route(const float* logits, int num_tokens, int experts, i
   PAE_REQUIRE(top > 0 && top <= keep * (experts / groups), "routing: %d experts chosen of %d that can be", top,
               keep * (experts / groups));
   if (num_tokens <= 0) return 0;
-  moe_route_kernel<<<num_tokens, PAE_WAVE, (size_t)(experts + groups + (choice_bias ? experts : 0)) * sizeof(float), stream>>>(
-      logits, experts, groups, keep, top, scale, choice_bias, ldz, among_chosen, shared_pieces, chosen, weights);
+  const size_t lds = (size_t)(experts + groups + (choice_bias ? experts : 0)) * sizeof(float);
+#define MOE_ROUTE(PER_LANE)                                                                                            \
+  moe_route_kernel<PER_LANE><<<num_tokens, PAE_WAVE, lds, stream>>>(logits, experts, groups, keep, top, scale, choice_bias, ldz, \
+                                                                    among_chosen, shared_pieces, chosen, weights)
+  if (experts <= PAE_WAVE) MOE_ROUTE(1);
+  else if (experts <= 4 * PAE_WAVE) MOE_ROUTE(4);
+  else MOE_ROUTE(MOE_MAX_PER_LANE);
+#undef MOE_ROUTE
   return pae_check_launch("moe_route");
 }
 

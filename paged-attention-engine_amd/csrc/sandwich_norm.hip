@@ -6,7 +6,8 @@
 //   normed = x / sqrt(mean(x^2) + eps_next) * w_next    (optional: the norm before the next sublayer)
 //   rows   = T(x)                                       (optional: the stream itself as a product's operand)
 //
-// A term is a sublayer's output [T, H] in the activation type, or float32 [T, H], or float32 partial sums
+// A term is a sublayer's output [T, H] in the activation type, or float32 [T, H], or one row [H] of either type that
+// every token adds (a bias), or float32 partial sums
 // [P, T, H] of a split product, which are added in order (two mixers side by side leave two terms with their
 // factors, routed experts one term of as many parts as a token has experts).  One workgroup a row; the row
 // waits in LDS between the passes, and a thread meets the same features in every pass.  Sums, both divisions
@@ -21,6 +22,7 @@ struct JoinTerms {
   int is_f32[PAE_JOIN_TERMS];
   int parts[PAE_JOIN_TERMS];
   int64_t part_stride[PAE_JOIN_TERMS];
+  int64_t row_stride[PAE_JOIN_TERMS];  // hidden, or 0 for one row that every token adds
   float scale[PAE_JOIN_TERMS];
   int count;
 };
@@ -77,7 +79,7 @@ __global__ __launch_bounds__(256) void norm_join_kernel(float* __restrict__ resi
       if (j >= terms.count) break;
       float sum[4] = {0.f, 0.f, 0.f, 0.f};
       if (terms.is_f32[j]) {
-        const float* p = (const float*)terms.ptr[j] + base + i;
+        const float* p = (const float*)terms.ptr[j] + blockIdx.x * terms.row_stride[j] + i;
         for (int part = 0; part < terms.parts[j]; ++part) {
           float t[4] = {0.f, 0.f, 0.f, 0.f};
           if (VEC) join_load4<float>(p + part * terms.part_stride[j], t);
@@ -86,7 +88,7 @@ __global__ __launch_bounds__(256) void norm_join_kernel(float* __restrict__ resi
           for (int e = 0; e < W; ++e) sum[e] += t[e];
         }
       } else {
-        const T* p = (const T*)terms.ptr[j] + base + i;
+        const T* p = (const T*)terms.ptr[j] + blockIdx.x * terms.row_stride[j] + i;
         if (VEC) join_load4<T>(p, sum);
         else sum[0] = to_f32(p[0]);
       }
@@ -136,7 +138,8 @@ __global__ __launch_bounds__(256) void norm_join_kernel(float* __restrict__ resi
 }
 
 extern "C" int pae_norm_join(int dtype, float* residual, int num_terms, const void* const* term_ptr, const int* term_is_f32,
-                             const int* term_parts, const int64_t* term_part_stride, const float* term_scale,
+                             const int* term_parts, const int64_t* term_part_stride, const int* term_one_row,
+                             const float* term_scale,
                              const void* w_out, int w_out_is_f32, float eps, const void* w_next, int w_next_is_f32,
                              float eps_next, void* normed, void* rows, int num_rows, int hidden, hipStream_t stream) {
   PAE_REQUIRE(num_terms >= 0 && num_terms <= PAE_JOIN_TERMS, "norm and join: %d terms (at most %d)", num_terms, PAE_JOIN_TERMS);
@@ -151,6 +154,7 @@ extern "C" int pae_norm_join(int dtype, float* residual, int num_terms, const vo
     terms.is_f32[j] = 0;
     terms.parts[j] = 1;
     terms.part_stride[j] = 0;
+    terms.row_stride[j] = hidden;
     terms.scale[j] = 0.f;
   }
   for (int j = 0; j < num_terms; ++j) {
@@ -159,6 +163,7 @@ extern "C" int pae_norm_join(int dtype, float* residual, int num_terms, const vo
     terms.is_f32[j] = term_is_f32[j];
     terms.parts[j] = term_parts[j];
     terms.part_stride[j] = term_part_stride[j];
+    terms.row_stride[j] = term_one_row[j] ? 0 : hidden;
     terms.scale[j] = term_scale[j];
   }
   const size_t lds = 2 * (size_t)hidden * sizeof(float);

@@ -103,7 +103,7 @@ def _declare(lib) -> None:
         "pae_sum_norm2": [I, P, I, P, P, P, P, P, P, I, P, I, F, P, P, P, I, I, I, P],
         "pae_project_f32": [I, P, L, P, L, P, P, I, I, I, I, P],
         "pae_moe_route": [P, I, I, I, I, I, F, P, L, I, I, P, P, P],
-        "pae_norm_join": [I, P, I, P, P, P, P, P, P, I, F, P, I, F, P, P, I, I, P],
+        "pae_norm_join": [I, P, I, P, P, P, P, P, P, P, I, F, P, I, F, P, P, I, I, P],
         "pae_linear_attention_step": [I, P, L, P, L, P, I, F, P, L, I, I, I, P, P, I, I, I, P, L, P, I, F, P, P, P],
         "pae_fixed_decay_chunk": [I],
         "pae_fixed_decay_step": [I, P, L, P, L, I, I, I, P, I, P, I, P, I, P, P, I, I, I, P, L, P, I, F, P, P, P],
@@ -1664,7 +1664,7 @@ def norm_join(residual: torch.Tensor, terms, w_out: Optional[torch.Tensor], eps:
               w_next: Optional[torch.Tensor] = None, eps_next: float = 0.0, normed: Optional[torch.Tensor] = None,
               rows: Optional[torch.Tensor] = None) -> None:
     """A sublayer's output joins the stream through the norm after it: y = sum of scale * term over `terms` (as for
-    `sum_norm2`), residual += y / sqrt(mean(y^2) + eps) * w_out (`w_out` None: residual += y), all float32.  Then,
+    `sum_norm2`; a term may also be one row [H] that every token adds), residual += y / sqrt(mean(y^2) + eps) * w_out (`w_out` None: residual += y), all float32.  Then,
     as asked: `normed` = residual / sqrt(mean(residual^2) + eps_next) * w_next, the norm before the next sublayer,
     and `rows` = the new residual itself, both in the activation type."""
     _not_while_recording("norm_join")
@@ -1680,22 +1680,23 @@ def norm_join(residual: torch.Tensor, terms, w_out: Optional[torch.Tensor], eps:
     assert w_out is None or w_out.numel() == H
     ptrs = (c_void_p * MAX_SUM_TERMS)()
     is_f32, parts = (c_int * MAX_SUM_TERMS)(), (c_int * MAX_SUM_TERMS)()
-    strides, scales = (c_int64 * MAX_SUM_TERMS)(), (c_float * MAX_SUM_TERMS)()
+    strides, scales, one_row = (c_int64 * MAX_SUM_TERMS)(), (c_float * MAX_SUM_TERMS)(), (c_int * MAX_SUM_TERMS)()
     for j, (t, scale) in enumerate(terms):
-        assert t.is_contiguous() and tuple(t.shape[-2:]) == (T, H)
+        assert t.is_contiguous() and (tuple(t.shape[-2:]) == (T, H) or tuple(t.shape) == (H,))
         if t.dim() == 3:
             assert t.dtype == torch.float32
         else:
-            assert t.dim() == 2
+            assert t.dim() in (1, 2)
             if t.dtype != torch.float32:
                 assert dtype is None or t.dtype == dtype
                 dtype = t.dtype
         ptrs[j], is_f32[j] = t.data_ptr(), 1 if t.dtype == torch.float32 else 0
         parts[j], strides[j], scales[j] = (t.shape[0] if t.dim() == 3 else 1), residual.numel(), float(scale)
+        one_row[j] = 1 if t.dim() == 1 else 0
     po, fo = _param(w_out)
     pn, fn = _param(w_next)
     _check(library().pae_norm_join(code_of(dtype or torch.float32), residual.data_ptr(), len(terms), ptrs, is_f32, parts,
-                                   strides, scales, po, fo, float(eps), pn, fn, float(eps_next), _ptr(normed), _ptr(rows),
+                                   strides, one_row, scales, po, fo, float(eps), pn, fn, float(eps_next), _ptr(normed), _ptr(rows),
                                    T, H, _stream()))
 
 

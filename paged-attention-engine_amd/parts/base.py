@@ -105,7 +105,7 @@ class ResidualStream:
 class BranchTerms(list):
     """What a block's branches leave pending on the stream when there are several of them: a list of
     (tensor, factor), each tensor [T, H] in the activation type or float32, or float32 partial sums
-    [P, T, H]; the norm that reads the stream next adds factor * tensor for each, in order, in float32.
+    [P, T, H] (where the block says so, `StepContext.takes_bias_terms`, also one row [H] that every token adds); the norm that reads the stream next adds factor * tensor for each, in order, in float32.
     A mixer that is several mixers side by side may return one as its output."""
 
 
@@ -177,6 +177,7 @@ class StepContext:
     cache_entry: int = 0               # the stop whose cache is read (entry itself unless it borrows)
     writes_cache: bool = True
     sink: Optional["BranchSink"] = None  # set by the block around a branch: see BranchSink
+    takes_bias_terms: bool = False     # set by the block around a branch: its output may be `BranchTerms` with a bias among them
     # room for the step's layers as one resident kernel (kernels.lib.DecodeProgram), offered by the step
     # function for steps in which every sequence brings one token; None: every kernel is launched by itself
     program: Optional[object] = None

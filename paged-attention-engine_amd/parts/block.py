@@ -463,7 +463,7 @@ class SandwichBlock:
     def forward(self, ctx, stream: ResidualStream) -> None:
         if stream.pending is not None or stream.owed is not None or stream.copies != 1:
             raise ValueError("a block with norms around its sublayers follows one that left the stream in another form")
-        ctx.sink = None
+        ctx.sink, ctx.takes_bias_terms = None, True
         prepared, stream.prepared = stream.prepared, None
         x = prepared[1] if prepared is not None and prepared[0] is self.mixer_norm else self.mixer_norm.forward(stream)
         follows = self._next_first_norm(stream)
@@ -482,6 +482,7 @@ class SandwichBlock:
             x, _ = self._join(stream, y, self.side.weight, self.side.eps, follows)
         if follows is not None:
             stream.prepared = (follows, x)
+        ctx.takes_bias_terms = False
 
 
 def build_block(layer_spec, dtype, device):

@@ -19,7 +19,7 @@ from typing import Optional
 import torch
 
 from ..kernels import lib as K
-from .base import OwedRows
+from .base import BranchTerms, OwedRows
 
 
 def rows_a_graph_may_hold(dtype: torch.dtype, *inner_sizes: int):
@@ -80,12 +80,17 @@ class Linear:
             return None
         return self._library(x, with_bias=False)
 
-    def branch(self, x: torch.Tensor, sink=None) -> Optional[torch.Tensor]:
+    def branch(self, x: torch.Tensor, sink=None, bias_terms: bool = False):
         """The product as a residual branch's output: [M, N] in x's dtype (few rows with a bias: k ranges
         that are added up inside the kernel, see `whole_sum_splits`), or float32
         partial sums [P, M, N] that the next norm adds up in order (no bias then).  With a `sink`
         whose norm can be folded, the few-row product adds itself into the residual instead and
-        prepares the following product's rows; nothing is returned then."""
+        prepares the following product's rows; nothing is returned then.  `bias_terms`: the consumer takes
+        `BranchTerms` with a bias among them (bfloat16: the product's partial sums or the library's plain
+        product, and the bias beside it, which the consumer adds in float32)."""
+        if bias_terms and self.bias is not None and x.dtype == torch.bfloat16 and x.shape[0]:
+            plain = Linear(self.weight)
+            return BranchTerms([(plain.branch(x), 1.0), (self.bias, 1.0)])
         if x.dtype == torch.bfloat16 and self.bias is None and x.shape[0] and K.skinny_supported(x, self.weight):
             splits = K.skinny_splits(self.out_features, self.in_features, x.shape[0])
             fold = sink.folded(x.shape[0]) if sink is not None else None

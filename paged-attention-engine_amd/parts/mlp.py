@@ -122,4 +122,4 @@ class DenseFeedForward(Part):
             if act is None:
                 act = self.up(x)
             K.activation(act, self.spec.activation, bias)
-        return self.down.branch(act, getattr(ctx, "sink", None))
+        return self.down.branch(act, getattr(ctx, "sink", None), getattr(ctx, "takes_bias_terms", False))

@@ -317,6 +317,9 @@ def test_gates_formed_from_the_mixers_input(dtype, hidden):
 class Context:
     sink = None
 
+    def __init__(self, takes_bias_terms=False):
+        self.takes_bias_terms = takes_bias_terms
+
 
 def part_of(spec, weights, dtype):
     from paged_attention_engine_amd.parts import FEED_FORWARDS, build_part
@@ -328,6 +331,9 @@ def part_of(spec, weights, dtype):
 
 
 def total(y):
+    """A branch's output, whatever form it came in, as one tensor."""
+    if isinstance(y, list):
+        return sum(factor * total(term) for term, factor in y)
     return y.double().sum(0) if y.dim() == 3 else y.double()
 
 
@@ -347,7 +353,27 @@ def test_dense_with_biases_and_the_square_of_relu(dtype, case):
     for T in (1, 5, 17, 64, 65, 200):
         x = draw(T, H).to(dtype)
         want = plain.dense(weights, "f.", x.double(), torch.float64)
-        close(total(part.forward(Context(), x.to(DEV))), want, 1e-5 if dtype == torch.float32 else 2e-2, f"{T} rows {case}")
+        for takes in (False, True):  # the second product's bias inside the product, or left to the norm that follows
+            y = part.forward(Context(takes), x.to(DEV))
+            assert isinstance(y, list) == (takes and dtype == torch.bfloat16)
+            close(total(y), want, 1e-5 if dtype == torch.float32 else 2e-2, f"{T} rows {case}")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H", [48, 90, 1536])
+def test_a_product_and_its_bias_join_through_offset_norms(dtype, H):
+    """x <- x + (1 + w) * normed(parts + bias), and the norm before the next sublayer, whose weight is stored around zero too."""
+    gen = torch.Generator().manual_seed(H)
+    T, eps = 9, 1e-4
+    x, parts = torch.randn((T, H), generator=gen), torch.randn((3, T, H), generator=gen)
+    bias = torch.randn(H, generator=gen).to(dtype)
+    w_out, w_next = torch.randn(H, generator=gen) * 0.3, torch.randn(H, generator=gen) * 0.3
+    y = parts.double().sum(0) + bias.double()
+    new = x.double() + plain.offset_norm(y, w_out.double(), eps)
+    residual, normed = x.to(DEV), torch.empty((T, H), dtype=dtype, device=DEV)
+    K().norm_join(residual, [(parts.to(DEV), 1.0), (bias.to(DEV), 1.0)], (1 + w_out).to(DEV), eps, (1 + w_next).to(DEV), eps, normed)
+    close(residual, new, 2e-6, "the new stream")
+    close(normed, plain.offset_norm(new, w_next.double(), eps), 1e-5 if dtype == torch.float32 else 1e-2, "the next norm")
 
 
 @pytest.mark.parametrize("case", [dict(E=6, top=2), dict(E=9, top=1), dict(E=4, top=4), dict(E=64, top=6), dict(E=200, top=8), dict(E=1, top=1)])
